@@ -45,11 +45,13 @@ attn_mfma_kernel(const __bf16* __restrict__ q, const __bf16* __restrict__ k_cach
                  const int32_t* __restrict__ positions, __bf16* __restrict__ out, float* __restrict__ part_o,
                  float* __restrict__ part_ml, int n_tiles, int n_splits, int heads, int kv_heads, int page_size,
                  int max_blocks, float scale_log2, int window, int page_shift, const float* __restrict__ sink,
-                 const float2* __restrict__ turn_back) {
+                 const float2* __restrict__ turn_back, float cap_slope, float cap2, const __bf16* __restrict__ gate,
+                 int64_t gate_stride) {
   // sink (one float per head, or null): exp(sink) joins the softmax's denominator, with no key and no value, not
   // scaled, once: the first slice's running maximum starts there with a sum of one.  turn_back ((cos, sin) per token
   // and pair, [tokens][D / 2], or null; D a multiple of 32): the result is rotated by minus these angles, element i
-  // with i + D / 2, which a lane holds both of.
+  // with i + D / 2, which a lane holds both of.  cap2 > 0: scores are capped (`ix_capped_log2`) before the mask.  gate
+  // (or null): the result of (token, head) is multiplied by the sigmoid of D numbers at gate_stride a token.
   constexpr int D = 16 * NB;
   constexpr int NC = (NB + 1) / 2;  // 32-wide chunks of the head dimension
   const int lane = threadIdx.x & 63;
@@ -203,6 +205,13 @@ attn_mfma_kernel(const __bf16* __restrict__ q, const __bf16* __restrict__ k_cach
       // scores stay unscaled: the scale (times log2 e) enters with the reference point in one fused multiply-add
       float sv[8];
       float mx = -INFINITY;
+      const float sl = cap2 > 0.f ? 1.0f : scale_log2;
+      if (cap2 > 0.f) {  // (uniform; capped scores are in units of log2 already)
+#pragma unroll
+        for (int b = 0; b < 2; ++b)
+#pragma unroll
+          for (int i = 0; i < 4; ++i) s[b][i] = ix_capped_log2(s[b][i], cap_slope, cap2);
+      }
       // keys that every query of these sixteen sees need no mask (uniform over the wavefront)
       // (GQ: the columns without a query head hold zeros for q; what they sum is not stored)
       const bool inner = (GQ || 16 * t + 16 <= rows) && kb + ATTN_KEYS_PER_ITER <= ke &&
@@ -228,7 +237,7 @@ attn_mfma_kernel(const __bf16* __restrict__ q, const __bf16* __restrict__ k_cach
       // The reference point m of the exponentials (in units of log2) follows the running maximum lazily: it moves
       // only when some query's maximum has outgrown it by more than 2^8, so the accumulators are seldom rescaled.
       // Any m gives the same quotient; probabilities up to 2^8 keep the relative precision of bfloat16.
-      const float top = mx * scale_log2;
+      const float top = mx * sl;
       if (__any(top > m[t] + 8.f)) {
         const float m_new = fmaxf(m[t], top);
         // v_exp_f32 as it is: a result below the smallest normal number may become 0
@@ -243,7 +252,7 @@ attn_mfma_kernel(const __bf16* __restrict__ q, const __bf16* __restrict__ k_cach
       bf16x8 pf;
 #pragma unroll
       for (int j = 0; j < 8; ++j) {
-        const float p = __builtin_amdgcn_exp2f(fmaf(sv[j], scale_log2, -m_safe));
+        const float p = __builtin_amdgcn_exp2f(fmaf(sv[j], sl, -m_safe));
         psum += p;
         pf[j] = (__bf16)p;
       }
@@ -281,8 +290,14 @@ attn_mfma_kernel(const __bf16* __restrict__ q, const __bf16* __restrict__ k_cach
 #pragma unroll
       for (int b = 0; b < NB; ++b) {
         bf16x4 v;
+        f32x4 by = f32x4{inv, inv, inv, inv};
+        if (gate) {
+          const bf16x4 gv = *reinterpret_cast<const bf16x4*>(gate + token * gate_stride + head * D + 4 * g + 16 * b);
 #pragma unroll
-        for (int i = 0; i < 4; ++i) v[i] = (__bf16)(o[t][b][i] * inv);
+          for (int i = 0; i < 4; ++i) by[i] = inv * __builtin_amdgcn_rcpf(1.0f + __expf(-(float)gv[i]));
+        }
+#pragma unroll
+        for (int i = 0; i < 4; ++i) v[i] = (__bf16)(o[t][b][i] * by[i]);
         *reinterpret_cast<bf16x4*>(dst + 16 * b) = v;
       }
     } else {
@@ -303,7 +318,8 @@ attn_mfma_kernel(const __bf16* __restrict__ q, const __bf16* __restrict__ k_cach
 // sums its columns with independent loads.
 __global__ void __launch_bounds__(128)
 attn_combine_kernel(const float* __restrict__ part_o, const float* __restrict__ part_ml, __bf16* __restrict__ out,
-                    int n_splits, int head_dim, int heads, const float2* __restrict__ turn_back) {
+                    int n_splits, int head_dim, int heads, const float2* __restrict__ turn_back,
+                    const __bf16* __restrict__ gate, int64_t gate_stride) {
   __shared__ float wgt[256];
   __shared__ float inv_l;
   const int64_t th = blockIdx.x;  // token * heads + head
@@ -324,6 +340,8 @@ attn_combine_kernel(const float* __restrict__ part_o, const float* __restrict__ 
   }
   __syncthreads();
   const float* po = part_o + th * n_splits * head_dim;
+  const __bf16* gr = gate ? gate + (th / heads) * gate_stride + (th % heads) * head_dim : nullptr;
+  auto gated = [&](float o, int d) { return gr ? o / (1.0f + __expf(-(float)gr[d])) : o; };
   if (turn_back) {  // the result rotated by minus the token's angles: a thread takes element d and d + head_dim / 2
     const int half = head_dim / 2;
     for (int d = threadIdx.x; d < half; d += blockDim.x) {
@@ -334,8 +352,8 @@ attn_combine_kernel(const float* __restrict__ part_o, const float* __restrict__ 
         w += wgt[s] * po[s * head_dim + half + d];
       }
       const float2 c = turn_back[(th / heads) * half + d];
-      out[th * head_dim + d] = (__bf16)((u * c.x + w * c.y) * inv_l);
-      out[th * head_dim + half + d] = (__bf16)((w * c.x - u * c.y) * inv_l);
+      out[th * head_dim + d] = (__bf16)gated((u * c.x + w * c.y) * inv_l, d);
+      out[th * head_dim + half + d] = (__bf16)gated((w * c.x - u * c.y) * inv_l, half + d);
     }
     return;
   }
@@ -343,14 +361,16 @@ attn_combine_kernel(const float* __restrict__ part_o, const float* __restrict__ 
     float acc = 0.f;
 #pragma unroll 8
     for (int s = 0; s < n_splits; ++s) acc += wgt[s] * po[s * head_dim + d];
-    out[th * head_dim + d] = (__bf16)(acc * inv_l);
+    out[th * head_dim + d] = (__bf16)gated(acc * inv_l, d);
   }
 }
 
 int ix_attention_combine(const float* part_o, const float* part_ml, void* out, int64_t tokens, int heads,
-                         int n_splits, int head_dim, hipStream_t stream, const float* turn_back) {
+                         int n_splits, int head_dim, hipStream_t stream, const float* turn_back, const void* gate,
+                         int64_t gate_stride) {
   hipLaunchKernelGGL(attn_combine_kernel, dim3(static_cast<unsigned>(tokens * heads)), dim3(128), 0, stream, part_o,
-                     part_ml, (__bf16*)out, n_splits, head_dim, heads, reinterpret_cast<const float2*>(turn_back));
+                     part_ml, (__bf16*)out, n_splits, head_dim, heads, reinterpret_cast<const float2*>(turn_back),
+                     (const __bf16*)gate, gate_stride);
   return ix_check_launch("ix_attention_combine");
 }
 
@@ -359,7 +379,8 @@ static void launch_attn(dim3 grid, hipStream_t stream, const void* q, const void
                         const int32_t* table, const int32_t* tile_seq, const int32_t* tile_q0,
                         const int32_t* tile_rows, const int32_t* positions, void* out, float* part_o, float* part_ml,
                         int n_tiles, int n_splits, int heads, int kv_heads, int page_size, int max_blocks,
-                        float scale_log2, int window, const float* sink, const float* turn_back) {
+                        float scale_log2, int window, const float* sink, const float* turn_back, float cap_slope,
+                        float cap2, const void* gate, int64_t gate_stride) {
   int page_shift = -1;  // log2 of the page size if it is a power of two
   for (int b = 4; b < 31; ++b)
     if (page_size == (1 << b)) page_shift = b;
@@ -371,7 +392,7 @@ static void launch_attn(dim3 grid, hipStream_t stream, const void* q, const void
   hipLaunchKernelGGL((attn_mfma_kernel<NB, QT, PF, GQ>), grid, dim3(64 * per_group), 0, stream, (const __bf16*)q, (const __bf16*)k,
                      (const __bf16*)v, table, tile_seq, tile_q0, tile_rows, positions, (__bf16*)out, part_o, part_ml,
                      n_tiles, n_splits, heads, kv_heads, page_size, max_blocks, scale_log2, window, page_shift, sink,
-                     reinterpret_cast<const float2*>(turn_back));
+                     reinterpret_cast<const float2*>(turn_back), cap_slope, cap2, (const __bf16*)gate, gate_stride);
 }
 
 // Workspace (when n_splits > 1): part_o float32 [tokens * heads * n_splits * head_dim],
@@ -383,7 +404,10 @@ static int attention_mfma_any(const void* q, const void* k_cache, const void* v_
                               const int32_t* positions, void* out, float* part_o, float* part_ml, int64_t tokens,
                               int n_tiles, int tile_queries, int n_splits, int heads, int kv_heads, int head_dim,
                               int page_size, int max_blocks, float scale, int window, int prefetch, int grouped,
-                              const float* sink, const float* turn_back, hipStream_t stream) {
+                              const float* sink, const float* turn_back, float softcap, const void* gate,
+                              int64_t gate_stride, hipStream_t stream) {
+  IX_REQUIRE(softcap >= 0.f, "the cap of the scores must not be negative");
+  IX_REQUIRE(gate == nullptr || gate_stride % 4 == 0, "a gate's rows must lie on 8-byte boundaries");
   IX_REQUIRE(turn_back == nullptr || head_dim % 32 == 0, "a result that is rotated back needs heads of a multiple of 32");
   IX_REQUIRE(tile_queries == 16 || tile_queries == 32, "a query tile holds up to 16 or 32 queries");
   IX_REQUIRE(tile_queries == 16 || head_dim <= 128, "tiles of 32 queries need head_dim <= 128");
@@ -401,9 +425,11 @@ static int attention_mfma_any(const void* q, const void* k_cache, const void* v_
   const int64_t units = static_cast<int64_t>(n_tiles) * n_splits;
   dim3 grid(static_cast<unsigned>((units + 3) / 4), grouped ? kv_heads : heads);
   const float scale_log2 = scale * 1.4426950408889634f;
+  const float cap2 = softcap * 1.4426950408889634f, cap_slope = softcap > 0.f ? 2.0f * scale_log2 / softcap : 0.f;
 #define ARGS                                                                                                    \
   grid, stream, q, k_cache, v_cache, block_table, tile_seq, tile_q0, tile_rows, positions, out, part_o, part_ml, \
-      n_tiles, n_splits, heads, kv_heads, page_size, max_blocks, scale_log2, window, sink, turn_back
+      n_tiles, n_splits, heads, kv_heads, page_size, max_blocks, scale_log2, window, sink, turn_back, cap_slope,    \
+      cap2, gate, gate_stride
 #define CASE(NB)                                                    \
   case NB:                                                          \
     if (grouped) {                                                  \
@@ -431,7 +457,8 @@ static int attention_mfma_any(const void* q, const void* k_cache, const void* v_
 #undef ARGS
   if (ix_check_launch("ix_attention_mfma")) return 1;
   if (n_splits > 1)
-    return ix_attention_combine(part_o, part_ml, out, tokens, heads, n_splits, head_dim, stream, turn_back);
+    return ix_attention_combine(part_o, part_ml, out, tokens, heads, n_splits, head_dim, stream, turn_back, gate,
+                                gate_stride);
   return 0;
 }
 
@@ -443,22 +470,23 @@ extern "C" int ix_attention_mfma(const void* q, const void* k_cache, const void*
                                  hipStream_t stream) {
   return attention_mfma_any(q, k_cache, v_cache, block_table, tile_seq, tile_q0, tile_rows, positions, out, part_o,
                             part_ml, tokens, n_tiles, tile_queries, n_splits, heads, kv_heads, head_dim, page_size,
-                            max_blocks, scale, window, prefetch, grouped, nullptr, nullptr, stream);
+                            max_blocks, scale, window, prefetch, grouped, nullptr, nullptr, 0.f, nullptr, 0, stream);
 }
 
 // The same with a sink per head (float32 [heads], or null) in every softmax's denominator, and with the result of
 // every (token, head) rotated back by the token's angles (turn_back float32 (cos, sin) [tokens, head_dim / 2], or
-// null; head_dim a multiple of 32).
+// null; head_dim a multiple of 32), with scores capped at softcap (0: not), and with the result multiplied by the
+// sigmoid of a gate (bfloat16 rows of heads * head_dim numbers, gate_stride apart, or null).
 extern "C" int ix_attention_mfma_sink(const void* q, const void* k_cache, const void* v_cache,
                                       const int32_t* block_table, const int32_t* tile_seq, const int32_t* tile_q0,
                                       const int32_t* tile_rows, const int32_t* positions, void* out, float* part_o,
                                       float* part_ml, int64_t tokens, int n_tiles, int tile_queries, int n_splits,
                                       int heads, int kv_heads, int head_dim, int page_size, int max_blocks, float scale,
                                       int window, int prefetch, int grouped, const float* sink, const float* turn_back,
-                                      hipStream_t stream) {
+                                      float softcap, const void* gate, int64_t gate_stride, hipStream_t stream) {
   return attention_mfma_any(q, k_cache, v_cache, block_table, tile_seq, tile_q0, tile_rows, positions, out, part_o,
                             part_ml, tokens, n_tiles, tile_queries, n_splits, heads, kv_heads, head_dim, page_size,
-                            max_blocks, scale, window, prefetch, grouped, sink, turn_back, stream);
+                            max_blocks, scale, window, prefetch, grouped, sink, turn_back, softcap, gate, gate_stride, stream);
 }
 
 // ---- the same operation without a workspace argument -----------------------------------------------------------

@@ -13,7 +13,8 @@
 // denominator also holds exp(sink[head]), which has no key and no value, is not scaled and counts once: the running
 // maximum starts there with a sum of one.  `turn_back` (float32 (cos, sin) [T, value_dim / 2], or null): the result
 // of every head is rotated by minus the query's angles, pair (i, i + value_dim / 2), before it is rounded (for
-// values that were cached rotated by their own positions).
+// values that were cached rotated by their own positions).  `softcap` c > 0: a score becomes c tanh(score / c) after
+// the scale, before the mask and the softmax.
 #include "common.h"
 
 #define ATTN_PLAIN_THREADS 256
@@ -24,7 +25,7 @@ attn_plain_kernel(const T* __restrict__ q, const T* __restrict__ k_cache, const 
                   const int32_t* __restrict__ block_table, const int32_t* __restrict__ seq_of_token,
                   const int32_t* __restrict__ positions, T* __restrict__ out, int heads, int kv_heads, int head_dim,
                   int value_dim, int page_size, int max_blocks, float scale, int window,
-                  const float* __restrict__ sink, const float2* __restrict__ turn_back) {
+                  const float* __restrict__ sink, const float2* __restrict__ turn_back, float softcap) {
   __shared__ float qs[256];
   __shared__ float sc[ATTN_PLAIN_THREADS];
   __shared__ int32_t pg[ATTN_PLAIN_THREADS];
@@ -54,6 +55,7 @@ attn_plain_kernel(const T* __restrict__ q, const T* __restrict__ k_cache, const 
       float dot = 0.f;
       for (int i = 0; i < head_dim; ++i) dot += qs[i] * ix_load(kr + i);
       s = dot * scale;
+      if (softcap > 0.f) s = softcap * tanhf(s / softcap);
     }
     pg[tid] = page;
     const float m_new = fmaxf(m, ix_block_max(s, red));
@@ -94,22 +96,23 @@ extern "C" int ix_attention_plain(const void* q, const void* k_cache, const void
                                   const int32_t* block_table, const int32_t* seq_of_token, const int32_t* positions,
                                   void* out, int64_t tokens, int heads, int kv_heads, int head_dim, int value_dim,
                                   int page_size, int max_blocks, float scale, int window, const float* sink,
-                                  const float* turn_back, hipStream_t stream) {
+                                  const float* turn_back, float softcap, hipStream_t stream) {
   IX_REQUIRE(tokens >= 0 && heads > 0 && kv_heads > 0 && page_size > 0 && max_blocks > 0, "sizes must be positive");
   IX_REQUIRE(heads % kv_heads == 0, "heads must be a multiple of kv_heads");
   IX_REQUIRE(head_dim > 0 && head_dim <= 256, "head_dim must be between 1 and 256");
   IX_REQUIRE(value_dim > 0 && value_dim <= 256, "value_dim must be between 1 and 256");
   IX_REQUIRE(window >= 0, "window must not be negative");
+  IX_REQUIRE(softcap >= 0.f, "the cap of the scores must not be negative");
   if (tokens == 0) return 0;
   dim3 grid(tokens, heads), block(ATTN_PLAIN_THREADS);
   if (dtype == IX_F32)
     hipLaunchKernelGGL(attn_plain_kernel<float>, grid, block, 0, stream, (const float*)q, (const float*)k_cache,
                        (const float*)v_cache, block_table, seq_of_token, positions, (float*)out, heads, kv_heads,
-                       head_dim, value_dim, page_size, max_blocks, scale, window, sink, (const float2*)turn_back);
+                       head_dim, value_dim, page_size, max_blocks, scale, window, sink, (const float2*)turn_back, softcap);
   else if (dtype == IX_BF16)
     hipLaunchKernelGGL(attn_plain_kernel<bf16_t>, grid, block, 0, stream, (const bf16_t*)q, (const bf16_t*)k_cache,
                        (const bf16_t*)v_cache, block_table, seq_of_token, positions, (bf16_t*)out, heads, kv_heads,
-                       head_dim, value_dim, page_size, max_blocks, scale, window, sink, (const float2*)turn_back);
+                       head_dim, value_dim, page_size, max_blocks, scale, window, sink, (const float2*)turn_back, softcap);
   else
     IX_REQUIRE(false, "dtype must be float32 or bfloat16");
   return ix_check_launch("ix_attention_plain");

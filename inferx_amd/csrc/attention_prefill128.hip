@@ -33,7 +33,9 @@
 // Masking, the lazily moving reference point of the exponentials, slices of a
 // tile's keys with their parts, pairs of units per workgroup and the rule that
 // values of keys that no query may read enter LDS as zeros are those of
-// attention_prefill.hip.
+// attention_prefill.hip.  Options: a sink per head (exp(sink) in the denominator, with no key and no value: the first
+// slice's running maximum starts there with a sum of one), scores capped before the mask (CAP, `ix_capped_log2`), and
+// a gate whose sigmoid multiplies the result.
 #include "common.h"
 
 typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
@@ -45,7 +47,7 @@ typedef float f32x16 __attribute__((ext_vector_type(16)));
 #define PW_QUERIES 128  // queries per workgroup
 #define PW_LOADERS 256  // threads that load
 
-template <int NB2>  // head_dim = 32 * NB2
+template <int NB2, bool CAP>  // head_dim = 32 * NB2
 __global__ void __launch_bounds__(512)
 attn_prefill128_kernel(const __bf16* __restrict__ q, const __bf16* k_cache, const __bf16* v_cache,
                        const int32_t* __restrict__ block_table, const int32_t* __restrict__ tile_seq,
@@ -53,7 +55,8 @@ attn_prefill128_kernel(const __bf16* __restrict__ q, const __bf16* k_cache, cons
                        const int32_t* __restrict__ pair_a, const int32_t* __restrict__ pair_b,
                        const int32_t* __restrict__ positions, __bf16* __restrict__ out, float* __restrict__ part_o,
                        float* __restrict__ part_ml, int n_splits, int heads, int kv_heads, int page_size,
-                       int max_blocks, float scale_log2, int window, int page_shift) {
+                       int max_blocks, float scale_log2, int window, int page_shift, const float* __restrict__ sink,
+                       float cap_slope, float cap2, const __bf16* __restrict__ gate, int64_t gate_stride) {
   constexpr int D = 32 * NB2;
   constexpr int NS = D / 16;                          // steps of 16 of the head dimension in K Q^T
   constexpr int RS = D <= 32 ? 4 : (D <= 64 ? 8 : 16);  // 16-byte pieces per LDS row of the key tile
@@ -254,7 +257,9 @@ attn_prefill128_kernel(const __bf16* __restrict__ q, const __bf16* k_cache, cons
     for (int b = 0; b < NB2; ++b)
 #pragma unroll
       for (int i = 0; i < 16; ++i) o[b][i] = 0.f;
-    float m = -INFINITY, lsum = 0.f;
+    const bool sunk = sink != nullptr && split == 0;
+    float m = sunk ? sink[head] * 1.4426950408889634f : -INFINITY;
+    float lsum = (sunk && h == 0) ? 1.f : 0.f;  // (a query's sum is spread over its two lanes)
     const int swap32 = (lane ^ 32) << 2;  // ds_bpermute address of the lane that holds the other keys of this query
     // operand places: key row 32 b + qn has the permutation of row qn (32 is a multiple of what it repeats after),
     // value row 32 b + qn that of row qn likewise
@@ -305,6 +310,13 @@ attn_prefill128_kernel(const __bf16* __restrict__ q, const __bf16* k_cache, cons
         // keys that every query of the wavefront sees need no mask (uniform)
         const bool inner = wq0 + 32 <= rows && kb + PW_KEYS - 1 <= wfirst && (window == 0 || kb > wlast - window);
         float mx = -INFINITY;
+        const float sl = CAP ? 1.0f : scale_log2;  // (capped scores are in units of log2 already)
+        if constexpr (CAP) {
+#pragma unroll
+          for (int b = 0; b < 2; ++b)
+#pragma unroll
+            for (int i = 0; i < 16; ++i) s[b][i] = ix_capped_log2(s[b][i], cap_slope, cap2);
+        }
         if (inner) {
 #pragma unroll
           for (int b = 0; b < 2; ++b)
@@ -325,7 +337,7 @@ attn_prefill128_kernel(const __bf16* __restrict__ q, const __bf16* k_cache, cons
         // The reference point m of the exponentials (in units of log2) follows the running maximum lazily: it moves
         // only when some query's maximum has outgrown it by more than 2^8, so the accumulators are seldom rescaled.
         // Scores stay unscaled: the scale (times log2 e) enters with the reference point in one fused multiply-add.
-        const float top = mx * scale_log2;
+        const float top = mx * sl;
         if (__any(top > m + 8.f)) {
           const float m_new = fmaxf(m, top);
           const float alpha = __builtin_amdgcn_exp2f(m - ((m_new == -INFINITY) ? 0.f : m_new));
@@ -345,7 +357,7 @@ attn_prefill128_kernel(const __bf16* __restrict__ q, const __bf16* k_cache, cons
         for (int g = 0; g < 4; ++g)
 #pragma unroll
           for (int j = 0; j < 8; ++j) {
-            const float p = __builtin_amdgcn_exp2f(fmaf(s[g >> 1][8 * (g & 1) + j], scale_log2, -m_safe));
+            const float p = __builtin_amdgcn_exp2f(fmaf(s[g >> 1][8 * (g & 1) + j], sl, -m_safe));
             psum += p;
             pf[g][j] = (__bf16)p;
           }
@@ -389,8 +401,15 @@ attn_prefill128_kernel(const __bf16* __restrict__ q, const __bf16* k_cache, cons
 #pragma unroll
       for (int c = 0; c < 4; ++c) {
         bf16x4 v;
+        f32x4 by = f32x4{inv, inv, inv, inv};
+        if (gate) {
+          const bf16x4 gv = *reinterpret_cast<const bf16x4*>(gate + static_cast<int64_t>(tq0 + wq0 + qn) * gate_stride +
+                                                             head * D + 4 * h + 32 * b + 8 * c);
 #pragma unroll
-        for (int e = 0; e < 4; ++e) v[e] = (__bf16)(o[b][4 * c + e] * inv);
+          for (int e = 0; e < 4; ++e) by[e] = inv * __builtin_amdgcn_rcpf(1.0f + __expf(-(float)gv[e]));
+        }
+#pragma unroll
+        for (int e = 0; e < 4; ++e) v[e] = (__bf16)(o[b][4 * c + e] * by[e]);
         *reinterpret_cast<bf16x4*>(dst + 32 * b + 8 * c) = v;
       }
   }  // the two units
@@ -404,7 +423,10 @@ extern "C" int ix_attention_prefill128(const void* q, const void* k_cache, const
                                        int n_pairs, const int32_t* positions, void* out, float* part_o,
                                        float* part_ml, int n_splits, int64_t tokens, int n_tiles, int heads,
                                        int kv_heads, int head_dim, int page_size, int max_blocks, float scale,
-                                       int window, hipStream_t stream) {
+                                       int window, const float* sink, float softcap, const void* gate,
+                                       int64_t gate_stride, hipStream_t stream) {
+  IX_REQUIRE(softcap >= 0.f, "the cap of the scores must not be negative");
+  IX_REQUIRE(gate == nullptr || gate_stride % 4 == 0, "a gate's rows must lie on 8-byte boundaries");
   IX_REQUIRE(n_tiles >= 0 && heads > 0 && kv_heads > 0 && max_blocks > 0, "sizes must be positive");
   IX_REQUIRE(heads % kv_heads == 0, "heads must be a multiple of kv_heads");
   IX_REQUIRE(head_dim % 32 == 0 && head_dim >= 32 && head_dim <= 128, "head_dim must be a multiple of 32 up to 128");
@@ -419,16 +441,22 @@ extern "C" int ix_attention_prefill128(const void* q, const void* k_cache, const
   while ((1 << page_shift) < page_size) ++page_shift;
   dim3 grid(static_cast<unsigned>(n_pairs) * heads);
   const float scale_log2 = scale * 1.4426950408889634f;
-#define CASE(NB2)                                                                                                    \
-  case NB2:                                                                                                          \
-    hipLaunchKernelGGL((attn_prefill128_kernel<NB2>), grid, dim3(512), 0, stream, (const __bf16*)q,                  \
-                       (const __bf16*)k_cache, (const __bf16*)v_cache, block_table, tile_seq, tile_q0, tile_rows,    \
-                       pair_a, pair_b, positions, (__bf16*)out, part_o, part_ml, n_splits, heads, kv_heads, page_size, \
-                       max_blocks, scale_log2, window, page_shift);                                                  \
+  const float cap2 = softcap * 1.4426950408889634f, cap_slope = softcap > 0.f ? 2.0f * scale_log2 / softcap : 0.f;
+#define RUN(NB2, CAP)                                                                                                \
+  hipLaunchKernelGGL((attn_prefill128_kernel<NB2, CAP>), grid, dim3(512), 0, stream, (const __bf16*)q,               \
+                     (const __bf16*)k_cache, (const __bf16*)v_cache, block_table, tile_seq, tile_q0, tile_rows,      \
+                     pair_a, pair_b, positions, (__bf16*)out, part_o, part_ml, n_splits, heads, kv_heads, page_size, \
+                     max_blocks, scale_log2, window, page_shift, sink, cap_slope, cap2, (const __bf16*)gate, gate_stride)
+#define CASE(NB2)                           \
+  case NB2:                                 \
+    if (softcap > 0.f) RUN(NB2, true);      \
+    else RUN(NB2, false);                   \
     break;
   switch (head_dim / 32) { CASE(1) CASE(2) CASE(3) CASE(4) }
 #undef CASE
+#undef RUN
   if (ix_check_launch("ix_attention_prefill128")) return 1;
-  if (n_splits > 1) return ix_attention_combine(part_o, part_ml, out, tokens, heads, n_splits, head_dim, stream);
+  if (n_splits > 1) return ix_attention_combine(part_o, part_ml, out, tokens, heads, n_splits, head_dim, stream, nullptr, gate,
+                                                gate_stride);
   return 0;
 }

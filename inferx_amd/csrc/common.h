@@ -135,6 +135,12 @@ __device__ __forceinline__ float ix_glu(float g, float u, float limit) {
   return g / (1.0f + e) * u;
 }
 
+// A score capped on its way into the softmax: c tanh(score / c), in units of log2 (c log2(e) = cap2), from the raw product
+// (times slope = 2 log2(e) scale / c): c (1 - 2 / (1 + e^(2 score / c))).  The absolute error is a few parts in 10^7 of c.
+__device__ __forceinline__ float ix_capped_log2(float raw, float slope, float cap2) {
+  return fmaf(-2.0f * cap2, __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(raw * slope)), cap2);
+}
+
 // bits of a router's selection mode
 #define IX_ROUTE_RENORMALIZE 1  // the chosen weights are divided by their sum
 #define IX_ROUTE_SIGMOID 2      // an expert's score is sigmoid(z) of its own logit instead of the softmax over all
@@ -145,9 +151,12 @@ __device__ __forceinline__ float ix_glu(float g, float u, float limit) {
 #include <string>
 void ix_set_error(const std::string& msg);
 // out[t, h, :] from the parts that kernels which cut keys into slices leave (attention_mfma.hip)
-// (turn_back: float32 (cos, sin) [tokens, head_dim / 2]; the result is rotated by minus these angles, or null)
+// (turn_back: float32 (cos, sin) [tokens, head_dim / 2]; the result is rotated by minus these angles, or null; gate:
+// bfloat16, token t's numbers for head h from gate + t * gate_stride + h * head_dim on; the result is multiplied by
+// their sigmoid, or null)
 int ix_attention_combine(const float* part_o, const float* part_ml, void* out, int64_t tokens, int heads,
-                         int n_splits, int head_dim, hipStream_t stream, const float* turn_back = nullptr);
+                         int n_splits, int head_dim, hipStream_t stream, const float* turn_back = nullptr,
+                         const void* gate = nullptr, int64_t gate_stride = 0);
 int ix_check_launch(const char* what);
 #define IX_REQUIRE(cond, msg)                          \
   do {                                                 \

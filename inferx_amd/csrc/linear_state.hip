@@ -7,7 +7,8 @@
 // number per head (`w_head`) and there is no correction.  That covers the generalized delta rule (w a decay per
 // channel, a = rate * unit key, b = unit key) and plain decayed linear attention (lightning attention: a constant
 // decay per head).  r, k, v come in the run's type, optionally through silu.  The state is float32, kept per
-// request slot as [heads][vdim][dim] (a column's rows side by side), and the whole recurrence is float32.
+// request slot as [heads][vdim][dim] (a column's rows side by side), and the whole recurrence is float32.  Optionally
+// r and k are rotated (the first 2 * half numbers of a head, number i with i + half, a table per token) and k is scaled.
 //
 // A column of S only ever meets its own value, so the work is spread over (request, head, column); the rows of a
 // column are shared by four neighbouring lanes whose partial sums meet through DPP.  A wavefront owns 16 columns
@@ -56,7 +57,8 @@ __device__ __forceinline__ void ls_open8(const ls_piece<bf16_t>& x, float (&o)[8
 }
 
 // R: rows of a column per lane (4 R >= dim).  VEC: dim = 4 R, R a multiple of 8 and everything on 16-byte boundaries,
-// so that a lane reads its part of the state and of every operand in 16-byte pieces.
+// so that a lane reads its part of the state and of every operand in 16-byte pieces (a rotation then needs half a multiple
+// of 8).  Requests that bring more than `max_rows` rows are left to others (0: none).
 template <typename T, int R, bool VEC>
 __global__ void __launch_bounds__(64)
 linear_state_kernel(const T* __restrict__ r, const T* __restrict__ k, const T* __restrict__ v, int64_t r_stride,
@@ -64,12 +66,13 @@ linear_state_kernel(const T* __restrict__ r, const T* __restrict__ k, const T* _
                     const float* __restrict__ w_head, const float* __restrict__ a_rows,
                     const float* __restrict__ b_rows, float* __restrict__ state, int64_t state_stride,
                     const int32_t* __restrict__ q_start, const int32_t* __restrict__ state_slots,
-                    float* __restrict__ out, int heads, int dim, int vdim, int silu) {
+                    float* __restrict__ out, int heads, int dim, int vdim, int silu, const float2* __restrict__ cos_sin,
+                    int half, float k_scale, int max_rows) {
   const int lane = threadIdx.x, part = lane & 3;
   const int col = blockIdx.x * 16 + (lane >> 2);
   const int head = blockIdx.y, seq = blockIdx.z;
   const int t0 = q_start[seq], t1 = q_start[seq + 1];
-  if (t1 <= t0) return;
+  if (t1 <= t0 || (max_rows > 0 && t1 - t0 > max_rows)) return;
   const bool live = col < vdim;
   const int row0 = part * R;
   float* sp = state + static_cast<int64_t>(state_slots[seq]) * state_stride +
@@ -96,10 +99,25 @@ linear_state_kernel(const T* __restrict__ r, const T* __restrict__ k, const T* _
         float x[8], y[8];
         ls_load8(r + t * r_stride + c + i, x);
         ls_load8(k + t * k_stride + c + i, y);
+        if (cos_sin && row0 + i < 2 * half) {  // eight numbers of the lower or of the upper half, and their partners
+          const bool low = row0 + i < half;
+          const int other = low ? half : -half;
+          float xo[8], yo[8];
+          ls_load8(r + t * r_stride + c + i + other, xo);
+          ls_load8(k + t * k_stride + c + i + other, yo);
+          const float2* cs = cos_sin + static_cast<int64_t>(t) * half + row0 + i - (low ? 0 : half);
+#pragma unroll
+          for (int e = 0; e < 8; ++e) {
+            const float2 a = cs[e];
+            const float sn = low ? -a.y : a.y;
+            x[e] = x[e] * a.x + xo[e] * sn;
+            y[e] = y[e] * a.x + yo[e] * sn;
+          }
+        }
 #pragma unroll
         for (int e = 0; e < 8; ++e) {
           rr[i + e] = silu ? ls_silu(x[e]) : x[e];
-          kk[i + e] = silu ? ls_silu(y[e]) : y[e];
+          kk[i + e] = silu ? ls_silu(y[e]) : y[e] * k_scale;
         }
       }
 #pragma unroll
@@ -121,7 +139,15 @@ linear_state_kernel(const T* __restrict__ r, const T* __restrict__ k, const T* _
       if (silu) {
         rr[i] = ls_silu(rr[i]);
         kk[i] = ls_silu(kk[i]);
+      } else if (cos_sin && ok && row0 + i < 2 * half) {
+        const bool low = row0 + i < half;
+        const int64_t o = c + (low ? half : -half);
+        const float2 a = cos_sin[static_cast<int64_t>(t) * half + row0 + i - (low ? 0 : half)];
+        const float sn = low ? -a.y : a.y;
+        rr[i] = rr[i] * a.x + ix_load(r + t * r_stride + o) * sn;
+        kk[i] = kk[i] * a.x + ix_load(k + t * k_stride + o) * sn;
       }
+      kk[i] *= k_scale;
       ww[i] = (ok && w_rows) ? w_rows[static_cast<int64_t>(t) * heads * dim + c] : wh;
       aa[i] = (ok && a_rows) ? a_rows[static_cast<int64_t>(t) * heads * dim + c] : 0.f;
       bb[i] = (ok && b_rows) ? b_rows[static_cast<int64_t>(t) * heads * dim + c] : 0.f;
@@ -386,13 +412,16 @@ extern "C" int ix_linear_state(const void* r, const void* k, const void* v, int 
                                int64_t k_stride, int64_t v_stride, const float* w_rows, const float* w_head,
                                const float* a_rows, const float* b_rows, float* state, int64_t state_stride,
                                const int32_t* q_start, const int32_t* state_slots, float* out, int64_t tokens,
-                               int requests, int heads, int dim, int vdim, int silu, hipStream_t stream) {
+                               int requests, int heads, int dim, int vdim, int silu, const float* cos_sin, int half,
+                               float k_scale, int max_rows, hipStream_t stream) {
   IX_REQUIRE(tokens >= 0 && requests > 0 && heads > 0 && dim > 0 && vdim > 0, "sizes must be positive");
   IX_REQUIRE(dim <= 256, "a head's keys hold at most 256 numbers");
   IX_REQUIRE((w_rows != nullptr) != (w_head != nullptr), "the decay comes per row and channel or per head");
   IX_REQUIRE((a_rows != nullptr) == (b_rows != nullptr), "the correction's two vectors come together");
   IX_REQUIRE(state_stride >= static_cast<int64_t>(heads) * dim * vdim, "a slot's state is too small");
   IX_REQUIRE(requests < 65536 && heads < 65536, "too many requests or heads for one launch");
+  IX_REQUIRE(half >= 0 && 2 * half <= dim && (half == 0 || cos_sin != nullptr), "the rotated pairs must fit into the head");
+  IX_REQUIRE((half == 0 && k_scale == 1.0f) || !silu, "either a rotation and a scale, or silu");
   if (tokens == 0) return 0;
   // steps that bring a request many rows: chunks through LDS, where a head's keys are 16 .. 128 numbers, the
   // operands come in the two usual combinations, and every row starts on a 16-byte boundary
@@ -407,7 +436,7 @@ extern "C" int ix_linear_state(const void* r, const void* k, const void* v, int 
     const bool aligned = (all & 15) == 0 && (r_stride * elt) % 16 == 0 && (k_stride * elt) % 16 == 0 && state_stride % 4 == 0;
     vec16 = aligned;
     if ((dtype == IX_F32 || dtype == IX_BF16) && (corr || none) && aligned && tokens >= 4 * static_cast<int64_t>(requests) &&
-        (dim == 16 || dim == 32 || dim == 64 || dim == 128)) {
+        half == 0 && k_scale == 1.0f && max_rows == 0 && (dim == 16 || dim == 32 || dim == 64 || dim == 128)) {
 #define CHUNKED(T, SP, RPL, CORR, THREADS)                                                                               \
   hipLaunchKernelGGL((linear_state_chunk_kernel<T, SP, RPL, CORR, (CORR ? (SP * RPL >= 128 ? 16 : 32) : 64), THREADS>),  \
                      dim3((vdim + THREADS / SP - 1) / (THREADS / SP), heads, requests), dim3(THREADS), 0, stream,        \
@@ -433,7 +462,9 @@ extern "C" int ix_linear_state(const void* r, const void* k, const void* v, int 
 #define LAUNCH(T, R, VEC)                                                                                          \
   hipLaunchKernelGGL((linear_state_kernel<T, R, VEC>), grid, block, 0, stream, (const T*)r, (const T*)k,             \
                      (const T*)v, r_stride, k_stride, v_stride, w_rows, w_head, a_rows, b_rows, state, state_stride, \
-                     q_start, state_slots, out, heads, dim, vdim, silu)
+                     q_start, state_slots, out, heads, dim, vdim, silu, half > 0 ? (const float2*)cos_sin : nullptr, half,  \
+                     k_scale, max_rows)
+  if (half % 8 != 0) vec16 = false;  // (a rotated piece of eight must lie in one half)
 #define PICK(T)                                              \
   if (vec16 && dim == 32) LAUNCH(T, 8, true);                \
   else if (vec16 && dim == 64) LAUNCH(T, 16, true);          \

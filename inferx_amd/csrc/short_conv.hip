@@ -12,6 +12,7 @@
 //   silu          y <- y * sigmoid(y)
 //   rotation      the first `rot_dims` elements of every q and k head, element i paired with i + rot_dims / 2, by the
 //                 (cos, sin) table of the step's tokens; computed in float32
+//   temperature   q <- q * (1 + coef * ln(floor((p + 1) / every) + 1)) at position p, before it is rounded
 //   destination   q always to `out_q` [T, q channels]; k and v either to `out_k`, `out_v` (plain rows) or into the
 //                 paged cache at the token's slot: keys [pages, k heads, page, head_dim], values transposed within a
 //                 page [pages, v heads, value_dim, page]
@@ -44,7 +45,14 @@ struct ConvArgs {
   int rot_dims, silu, page_size;
   int units_qk_head;       // units of one q or k head: head_dim - rot_dims / 2
   int units;               // all units of a token
+  const int32_t* positions;  // [T], read for the temperature only
+  float temp_coef, temp_every;  // (every 0: none)
 };
+
+// what the q channels of a row are multiplied by
+__device__ __forceinline__ float conv_temperature(const ConvArgs& a, int64_t row) {
+  return 1.0f + a.temp_coef * logf(floorf(static_cast<float>(a.positions[row] + 1) / a.temp_every) + 1.0f);
+}
 
 template <typename T>
 __device__ __forceinline__ float conv_input(const ConvArgs& a, const T* in, const float* st, int64_t row0, int x, int c) {
@@ -140,9 +148,10 @@ __global__ void __launch_bounds__(CONV_THREADS) short_conv_kernel(ConvArgs a) {
       break;
     }
     const int64_t row = row0 + ii;
-    float y0 = conv_at(a, in, st, row0, ii, c0);
+    const float temp = (a.temp_every > 0.f && c0 < a.q_channels) ? conv_temperature(a, row) : 1.0f;
+    float y0 = conv_at(a, in, st, row0, ii, c0) * temp;
     if (c1 >= 0) {
-      float y1 = conv_at(a, in, st, row0, ii, c1);
+      float y1 = conv_at(a, in, st, row0, ii, c1) * temp;
       if (a.cos_sin) {
         const float* cs = a.cos_sin + (row * (a.rot_dims / 2) + pair) * 2;
         const float c = cs[0], s = cs[1];
@@ -334,9 +343,14 @@ __global__ void __launch_bounds__(CONV_THREADS) short_conv_vec8_kernel(ConvArgs 
       break;
     }
     const int64_t row = row0 + ii;
+    const float temp = (a.temp_every > 0.f && c0 < a.q_channels) ? conv_temperature(a, row) : 1.0f;
     Conv8 y0 = conv_at8(a, wt, bias_f, in, st, row0, ii, c0);
+#pragma unroll
+    for (int e = 0; e < 8; ++e) y0.x[e] *= temp;
     if (c1 >= 0) {
       Conv8 y1 = conv_at8(a, wt, bias_f, in, st, row0, ii, c1);
+#pragma unroll
+      for (int e = 0; e < 8; ++e) y1.x[e] *= temp;
       if (a.cos_sin) {
         const float* cs = a.cos_sin + (row * (a.rot_dims / 2) + pair0) * 2;
 #pragma unroll
@@ -373,7 +387,7 @@ extern "C" int ix_short_conv(const void* in, int dtype, int64_t in_stride, const
                              const float* cos_sin, int rot_dims, int silu, const int32_t* slots, int page_size,
                              void* out_q, void* out_k, void* out_v, int64_t tokens, int q_channels, int k_channels,
                              int v_channels, int head_dim, int value_dim, const float* wt, const float* bias_f,
-                             hipStream_t stream) {
+                             const int32_t* positions, float temp_coef, float temp_every, hipStream_t stream) {
   IX_REQUIRE(tokens >= 0 && taps >= 1 && taps <= 64, "between 1 and 64 taps");
   IX_REQUIRE(head_dim > 0 && value_dim > 0 && q_channels >= 0 && k_channels >= 0 && v_channels >= 0,
              "sizes must be positive");
@@ -383,6 +397,7 @@ extern "C" int ix_short_conv(const void* in, int dtype, int64_t in_stride, const
   IX_REQUIRE(cos_sin != nullptr || rot_dims == 0, "a rotation needs its table");
   IX_REQUIRE(slots == nullptr || page_size > 0, "page_size must be positive");
   IX_REQUIRE(dtype == IX_F32 || dtype == IX_BF16, "dtype must be float32 or bfloat16");
+  IX_REQUIRE(temp_every >= 0.f && (temp_every == 0.f || positions != nullptr), "a temperature needs the rows' positions");
   const int channels = q_channels + k_channels + v_channels;
   IX_REQUIRE(in_stride >= channels && state_stride >= static_cast<int64_t>(taps - 1) * channels, "strides too small");
   if (tokens == 0 || channels == 0) return 0;
@@ -393,6 +408,7 @@ extern "C" int ix_short_conv(const void* in, int dtype, int64_t in_stride, const
   a.taps = taps; a.channels = channels; a.q_channels = q_channels; a.k_channels = k_channels; a.v_channels = v_channels;
   a.head_dim = head_dim; a.value_dim = value_dim; a.rot_dims = rot_dims; a.silu = silu; a.page_size = page_size;
   a.units_qk_head = head_dim - rot_dims / 2;
+  a.positions = positions; a.temp_coef = temp_coef; a.temp_every = temp_every;
   a.units = (q_channels + k_channels) / head_dim * a.units_qk_head + v_channels;
   IX_REQUIRE(tokens < (1ll << 31) && a.units <= 65535 * CONV_THREADS, "too many tokens or channels for one launch");
   dim3 grid(static_cast<unsigned>(tokens), (a.units + CONV_THREADS - 1) / CONV_THREADS), block(CONV_THREADS);

@@ -234,10 +234,12 @@ def _check_caches(q, k_cache, v_cache):
 
 def attention_plain(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, block_table: torch.Tensor,
                     seq_of_token: torch.Tensor, positions: torch.Tensor, out: torch.Tensor, scale: float,
-                    window: int, sink: Optional[torch.Tensor] = None, turn_back: Optional[torch.Tensor] = None) -> None:
+                    window: int, sink: Optional[torch.Tensor] = None, turn_back: Optional[torch.Tensor] = None,
+                    softcap: float = 0.0) -> None:
     """Paged attention, one workgroup per (token, head).  q [T, heads, d], out [T, heads, value size] (the value
     cache's).  `sink` float32 [heads]: exp(sink) joins every softmax's denominator, with no key and no value.
-    `turn_back` float32 [T, value size / 2, 2]: every head's result is rotated by minus these angles (halves paired)."""
+    `turn_back` float32 [T, value size / 2, 2]: every head's result is rotated by minus these angles (halves paired).
+    `softcap` c > 0: scores become c tanh(score / c)."""
     T, heads, d = q.shape
     vd = v_cache.shape[2]
     _need(out.shape == (T, heads, vd) and out.dtype == q.dtype, "out mismatch")
@@ -252,7 +254,7 @@ def attention_plain(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tenso
     _is_i32(positions, T)
     _call("ix_attention_plain", _ptr(q), _ptr(k_cache), _ptr(v_cache), _i32(_dt(q)), _ptr(block_table),
           _ptr(seq_of_token), _ptr(positions), _ptr(out), _i64(T), _i32(heads), _i32(kv_heads), _i32(d), _i32(vd),
-          _i32(page_size), _i32(block_table.shape[1]), _f32(scale), _i32(window), _ptr(sink), _ptr(turn_back), _stream())
+          _i32(page_size), _i32(block_table.shape[1]), _f32(scale), _i32(window), _ptr(sink), _ptr(turn_back), _f32(softcap), _stream())
 
 
 def qkv_norm_rope_append(qkv: torch.Tensor, q_norm: Optional[torch.Tensor], k_norm: Optional[torch.Tensor], eps: float,
@@ -310,7 +312,8 @@ def attention_mfma(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor
                    tiles: torch.Tensor, positions: torch.Tensor, out: torch.Tensor, n_splits: int,
                    workspace: Optional[torch.Tensor], scale: float, window: int, tile_queries: int = 16,
                    prefetch: bool = False, grouped: bool = False, sink: Optional[torch.Tensor] = None,
-                   turn_back: Optional[torch.Tensor] = None) -> None:
+                   turn_back: Optional[torch.Tensor] = None, softcap: float = 0.0,
+                   gate: Optional[torch.Tensor] = None) -> None:
     """Paged attention on the matrix cores (bfloat16).  `tiles` int32 [3, n_tiles]: request, first token row and
     number of rows (<= tile_queries, which is 16 or 32) of each query tile.  `workspace` float32 with T * heads * n_splits * (d + 2) entries
     when n_splits > 1.  `grouped`: every tile is ONE token, and the query heads of a key/value head (at most 16)
@@ -340,21 +343,34 @@ def attention_mfma(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor
             _i32(n_tiles), _i32(tile_queries), _i32(n_splits), _i32(heads), _i32(kv_heads), _i32(d), _i32(page_size),
             _i32(block_table.shape[1]), _f32(scale), _i32(window), _i32(1 if prefetch else 0),
             _i32(1 if grouped else 0))
-    if sink is None and turn_back is None:
+    if sink is None and turn_back is None and softcap <= 0 and gate is None:
         _call("ix_attention_mfma", *args, _stream())
         return
     # `sink` float32 [heads]: exp(sink) joins every softmax's denominator; `turn_back` float32 [T, d / 2, 2]: the
-    # result of every (token, head) is rotated by minus these angles, halves paired (d a multiple of 32)
+    # result of every (token, head) is rotated by minus these angles, halves paired (d a multiple of 32); `softcap` c > 0:
+    # scores become c tanh(score / c); `gate` [T, >= heads * d] rows: the result is multiplied by their sigmoid
     _need(sink is None or (sink.dtype == torch.float32 and sink.numel() == heads), "one float32 sink per head")
     _need(turn_back is None or (turn_back.dtype == torch.float32 and turn_back.shape == (T, d // 2, 2) and d % 32 == 0
                                 and turn_back.is_contiguous()), "turn_back must be float32 [T, d / 2, 2], d a multiple of 32")
-    _call("ix_attention_mfma_sink", *args, _ptr(sink), _ptr(turn_back), _stream())
+    gate_ptr, gate_stride = _gate_rows(gate, T, heads * d, q.dtype)
+    _call("ix_attention_mfma_sink", *args, _ptr(sink), _ptr(turn_back), _f32(softcap), gate_ptr, _i64(gate_stride), _stream())
+
+
+def _gate_rows(gate: Optional[torch.Tensor], tokens: int, width: int, dtype):
+    """(address, row stride) of a gate that an attention kernel applies to its result: rows of `width` numbers of the
+    activations' type on 8-byte boundaries."""
+    if gate is None:
+        return None, 0
+    _need(gate.dim() == 2 and gate.shape == (tokens, width) and gate.stride(1) == 1 and gate.dtype == dtype and gate.is_cuda
+          and gate.stride(0) % 4 == 0 and gate.data_ptr() % 8 == 0, "the gate must be rows of heads * head_dim numbers")
+    return gate.data_ptr(), gate.stride(0)
 
 
 def attention_prefill(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, block_table: torch.Tensor,
                       tiles: torch.Tensor, positions: torch.Tensor, out: torch.Tensor, scale: float, window: int,
                       tile_queries: int = 64, pairs: Optional[torch.Tensor] = None, n_splits: int = 1,
-                      workspace: Optional[torch.Tensor] = None) -> None:
+                      workspace: Optional[torch.Tensor] = None, sink: Optional[torch.Tensor] = None,
+                      softcap: float = 0.0, gate: Optional[torch.Tensor] = None) -> None:
     """Paged attention for prompt portions (bfloat16, head_dim <= 128): tiles of up to 64 queries of one
     request, keys and values shared through LDS; or, with `tile_queries` 128 (head_dim a multiple of 32), tiles of
     up to 128 queries, 32 per wavefront, with wavefronts of their own for the loads.  `tiles` as for attention_mfma.  `pairs` int32 [2, n]: the two
@@ -363,7 +379,9 @@ def attention_prefill(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Ten
 
     A unit is a tile, or with n_splits > 1 slice `unit % n_splits` of the keys of tile `unit // n_splits`; then
     `workspace` (float32, T * heads * n_splits * (d + 2) entries) takes the slices' parts, and ALL T rows of `out`
-    are written from it: rows that no tile covers get no meaningful values and are for the caller to fill."""
+    are written from it: rows that no tile covers get no meaningful values and are for the caller to fill.
+
+    `sink`, `softcap` and `gate` as for `attention_mfma`, for tiles of 128 queries only."""
     T, heads, d = q.shape
     _need(q.dtype == torch.bfloat16, "the matrix-core attention kernel is bfloat16 only")
     _need(out.shape == q.shape and out.dtype == q.dtype, "out mismatch")
@@ -391,12 +409,15 @@ def attention_prefill(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Ten
         part_ml = workspace[T * heads * n_splits * d:]
     if tile_queries == 128:
         _need(d % 32 == 0, "tiles of 128 queries take head sizes in steps of 32")
+        _need(sink is None or (sink.dtype == torch.float32 and sink.numel() == heads), "one float32 sink per head")
+        gate_ptr, gate_stride = _gate_rows(gate, T, heads * d, q.dtype)
         _call("ix_attention_prefill128", _ptr(q), _ptr(k_cache), _ptr(v_cache), _ptr(block_table), _ptr(tiles[0]),
               _ptr(tiles[1]), _ptr(tiles[2]), _ptr(pairs[0]), _ptr(pairs[1]), _i32(pairs.shape[1]), _ptr(positions),
               _ptr(out), _ptr(part_o), _ptr(part_ml), _i32(n_splits), _i64(T), _i32(tiles.shape[1]), _i32(heads),
               _i32(kv_heads), _i32(d), _i32(page_size), _i32(block_table.shape[1]), _f32(scale), _i32(window),
-              _stream())
+              _ptr(sink), _f32(softcap), gate_ptr, _i64(gate_stride), _stream())
         return
+    _need(sink is None and softcap <= 0 and gate is None, "sinks, capped scores and gates take tiles of 128 queries")
     _call("ix_attention_prefill", _ptr(q), _ptr(k_cache), _ptr(v_cache), _ptr(block_table), _ptr(tiles[0]),
           _ptr(tiles[1]), _ptr(tiles[2]), _ptr(pairs[0]), _ptr(pairs[1]), _i32(pairs.shape[1]), _ptr(positions),
           _ptr(out), _ptr(part_o), _ptr(part_ml), _i32(n_splits), _i64(T), _i32(tiles.shape[1]), _i32(tile_queries),
@@ -1068,7 +1089,7 @@ def short_conv(x: torch.Tensor, bias: Optional[torch.Tensor], weight: torch.Tens
                rows: StepRows, sizes: Tuple[int, int, int, int, int], out_q: torch.Tensor,
                out_k: torch.Tensor, out_v: torch.Tensor, slots: Optional[torch.Tensor] = None,
                cos_sin: Optional[torch.Tensor] = None, silu: bool = False, weight_t: Optional[torch.Tensor] = None,
-               bias_f32: Optional[torch.Tensor] = None) -> None:
+               bias_f32: Optional[torch.Tensor] = None, temperature: Optional[Tuple[torch.Tensor, float, float]] = None) -> None:
     """A causal convolution of `taps` = weight.shape[1] taps over time on the first q + k + v channels of x
     [T, >= channels] (a bias added first), continued from `state` (a float32 view [slots, >= (taps - 1) * channels]
     of each request's last inputs, brought up to date), then silu and / or the rotation of the first
@@ -1076,7 +1097,8 @@ def short_conv(x: torch.Tensor, bias: Optional[torch.Tensor], weight: torch.Tens
     value_dim).  With `slots` k and v go into the paged caches out_k [pages, k heads, page, head_dim] and out_v
     [pages, v heads, value_dim, page]; else to rows [T, k channels], [T, v channels].  q goes to out_q [T, q channels].
     `weight_t` float32 [taps, channels] and `bias_f32` float32 [channels]: the same numbers as `weight` and `bias`, laid
-    out for the kernel's 16-byte form (used where the sizes come in eights)."""
+    out for the kernel's 16-byte form (used where the sizes come in eights).  `temperature` = (positions [T], coef, every):
+    q is multiplied by 1 + coef ln(floor((position + 1) / every) + 1) before it is rounded."""
     cq, ck, cv, d, vd = sizes
     T = x.shape[0]
     C = cq + ck + cv
@@ -1105,11 +1127,16 @@ def short_conv(x: torch.Tensor, bias: Optional[torch.Tensor], weight: torch.Tens
         _need(weight_t.dtype == torch.float32 and weight_t.shape == (taps, C) and weight_t.is_contiguous(), "weight_t shape")
     if bias_f32 is not None:
         _need(bias_f32.dtype == torch.float32 and bias_f32.numel() == C and bias_f32.is_contiguous(), "bias_f32 shape")
+    positions, coef, every = temperature if temperature is not None else (None, 0.0, 0.0)
+    if positions is not None:
+        _is_i32(positions, T)
+        _need(every > 0, "the temperature's step must be positive")
     _call("ix_short_conv", x.data_ptr(), _i32(_dt(x)), _i64(x.stride(0)), _ptr(bias),
           _i32(_dt(bias) if bias is not None else F32), _ptr(weight), _i32(_dt(weight)), _i32(taps), state.data_ptr(),
           _i64(state.stride(0)), _ptr(rows.seq_of_token), _ptr(rows.q_start), _ptr(rows.state_slots), _ptr(cos_sin),
           _i32(rot), _i32(1 if silu else 0), _ptr(slots), _i32(page_size), _ptr(out_q), _ptr(out_k), _ptr(out_v),
-          _i64(T), _i32(cq), _i32(ck), _i32(cv), _i32(d), _i32(vd), _ptr(weight_t), _ptr(bias_f32), _stream())
+          _i64(T), _i32(cq), _i32(ck), _i32(cv), _i32(d), _i32(vd), _ptr(weight_t), _ptr(bias_f32), _ptr(positions), _f32(coef),
+          _f32(every), _stream())
 
 
 def delta_rule(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, ab: torch.Tensor, a_log: torch.Tensor,
@@ -1305,12 +1332,16 @@ def add_branches(h: torch.Tensor, a: torch.Tensor, b: Optional[torch.Tensor] = N
 def linear_state(r: torch.Tensor, k: torch.Tensor, v: torch.Tensor, state: torch.Tensor, rows: StepRows,
                  out: torch.Tensor, heads: int, dim: int, vdim: int, w_rows: Optional[torch.Tensor] = None,
                  w_head: Optional[torch.Tensor] = None, a_rows: Optional[torch.Tensor] = None,
-                 b_rows: Optional[torch.Tensor] = None, silu: bool = False) -> None:
+                 b_rows: Optional[torch.Tensor] = None, silu: bool = False, cos_sin: Optional[torch.Tensor] = None,
+                 k_scale: float = 1.0, max_rows: int = 0) -> None:
     """S <- diag(w) S - a (b^T S) + k v^T;  o = S^T r, over the rows of a step, request by request, from and to
     `state` (a float32 view [slots, >= heads * vdim * dim], a head's matrix kept [vdim][dim]).  r, k [T, heads * dim],
     v [T, heads * vdim] of the run's type (rows may be strided), through silu first if `silu`.  The decay w comes per
     row and key channel (`w_rows` float32 [T, heads * dim]) or per head (`w_head` float32 [heads]); the correction's
-    vectors `a_rows`, `b_rows` (float32 [T, heads * dim]) come together or not at all.  out float32 [T, heads, vdim]."""
+    vectors `a_rows`, `b_rows` (float32 [T, heads * dim]) come together or not at all.  out float32 [T, heads, vdim].
+    `cos_sin` float32 [T, half, 2]: the first 2 * half numbers of every head of r and k are rotated, number i with
+    i + half; then k is multiplied by `k_scale` (neither goes with silu).  `max_rows` > 0: requests that bring more rows
+    are left alone, their rows of `out` and their state too."""
     T = r.shape[0]
     for t, n in ((r, heads * dim), (k, heads * dim), (v, heads * vdim)):
         _need(t.dim() == 2 and t.shape == (T, n) and t.stride(1) == 1 and t.dtype == r.dtype and t.is_cuda, "r, k or v shape")
@@ -1324,11 +1355,56 @@ def linear_state(r: torch.Tensor, k: torch.Tensor, v: torch.Tensor, state: torch
           and state.shape[1] >= heads * dim * vdim, "the state must be float32 [slots, >= heads * dim * vdim]")
     _need(out.dtype == torch.float32 and out.shape == (T, heads, vdim) and out.is_contiguous(), "out must be float32 [T, heads, vdim]")
     rows.check(T)
+    half = _rotation_half(cos_sin, T, dim)
     S = rows.q_start.numel() - 1
     _call("ix_linear_state", r.data_ptr(), k.data_ptr(), v.data_ptr(), _i32(_dt(r)), _i64(r.stride(0)), _i64(k.stride(0)),
           _i64(v.stride(0)), _ptr(w_rows), _ptr(w_head), _ptr(a_rows), _ptr(b_rows), state.data_ptr(),
           _i64(state.stride(0)), _ptr(rows.q_start), _ptr(rows.state_slots), _ptr(out), _i64(T), _i32(S), _i32(heads),
-          _i32(dim), _i32(vdim), _i32(1 if silu else 0), _stream())
+          _i32(dim), _i32(vdim), _i32(1 if silu else 0), _ptr(cos_sin), _i32(half), _f32(k_scale), _i32(max_rows), _stream())
+
+
+def _rotation_half(cos_sin: Optional[torch.Tensor], tokens: int, dim: int) -> int:
+    """How many pairs of a head a rotation table turns (0 without one)."""
+    if cos_sin is None:
+        return 0
+    _need(cos_sin.dtype == torch.float32 and cos_sin.dim() == 3 and cos_sin.shape[0] == tokens and cos_sin.shape[2] == 2
+          and 2 * cos_sin.shape[1] <= dim and cos_sin.is_contiguous(), "the rotation table must be float32 [T, half, 2]")
+    return cos_sin.shape[1]
+
+
+LINEAR_CHUNK_ROWS = 64  # rows per chunk of `linear_chunks`
+
+
+def linear_chunks_fits(dim: int) -> bool:
+    return dim <= 128 and dim % 4 == 0
+
+
+def linear_chunks(r: torch.Tensor, k: torch.Tensor, v: torch.Tensor, state: torch.Tensor, state_slots: torch.Tensor,
+                  chunks: torch.Tensor, seqs: torch.Tensor, out: torch.Tensor, heads: int, dim: int, vdim: int,
+                  w_head: torch.Tensor, silu: bool = False, cos_sin: Optional[torch.Tensor] = None,
+                  k_scale: float = 1.0) -> None:
+    """`linear_state` with a decay per head, for the requests that `seqs` names, their rows cut into chunks that are worked
+    at the same time.  `chunks` int32 [2, n]: first row in the step and rows (1 .. LINEAR_CHUNK_ROWS) of every chunk;
+    `seqs` int32 [3, m]: the request, its first chunk, its number of chunks (at least one, in the order of its rows)."""
+    T = r.shape[0]
+    for t, n in ((r, heads * dim), (k, heads * dim), (v, heads * vdim)):
+        _need(t.dim() == 2 and t.shape == (T, n) and t.stride(1) == 1 and t.dtype == r.dtype and t.is_cuda, "r, k or v shape")
+    _need(w_head.dtype == torch.float32 and w_head.numel() == heads, "w_head must be float32 [heads]")
+    _need(state.dtype == torch.float32 and state.dim() == 2 and state.stride(1) == 1
+          and state.shape[1] >= heads * dim * vdim, "the state must be float32 [slots, >= heads * dim * vdim]")
+    _need(out.dtype == torch.float32 and out.shape == (T, heads, vdim) and out.is_contiguous(), "out must be float32 [T, heads, vdim]")
+    _need(linear_chunks_fits(dim), "a head's keys: a multiple of four numbers, at most 128")
+    _is_i32(state_slots)
+    for t, n in ((chunks, 2), (seqs, 3)):
+        _is_i32(t)
+        _need(t.dim() == 2 and t.shape[0] == n and t.is_contiguous(), "chunks int32 [2, n], seqs int32 [3, m]")
+    half = _rotation_half(cos_sin, T, dim)
+    kv = torch.empty((chunks.shape[1], heads, vdim, dim), dtype=torch.float32, device=r.device)
+    _call("ix_linear_chunks", r.data_ptr(), k.data_ptr(), v.data_ptr(), _i32(_dt(r)), _i64(r.stride(0)), _i64(k.stride(0)),
+          _i64(v.stride(0)), _ptr(w_head), _ptr(cos_sin), _i32(half), _f32(k_scale), _i32(1 if silu else 0), state.data_ptr(),
+          _i64(state.stride(0)), _ptr(state_slots), _ptr(chunks[0]), _ptr(chunks[1]), _i32(chunks.shape[1]), _ptr(seqs[0]),
+          _ptr(seqs[1]), _ptr(seqs[2]), _i32(seqs.shape[1]), _ptr(kv), _ptr(out), _i32(heads), _i32(dim), _i32(vdim),
+          _stream())
 
 
 def delta_operands(w_logit: torch.Tensor, w_bias: torch.Tensor, a_logit: torch.Tensor, a_bias: torch.Tensor,
@@ -1353,6 +1429,50 @@ def tanh_(x: torch.Tensor) -> None:
     """x = tanh(x) in place, float32."""
     _need(x.dtype == torch.float32 and x.is_contiguous(), "x must be float32")
     _call("ix_tanh_inplace", _ptr(x), _i64(x.numel()), _stream())
+
+
+# ---- a residual stream kept in several copies --------------------------------------------------------------------------
+def embed_norm(h: torch.Tensor, table: torch.Tensor, ids: torch.Tensor, weight: Optional[torch.Tensor], eps: float,
+               scale: float = 1.0) -> None:
+    """h [T, streams, W] float32: every copy of row t is rmsnorm(table[ids[t]] * scale) * weight (without a weight the
+    row as it is)."""
+    T, S, W = h.shape
+    _need(h.dtype == torch.float32, "the residual stream is float32")
+    _need(table.dim() == 2 and table.shape[1] == W, "table width differs from h")
+    _is_i32(ids, T)
+    _call("ix_embed_norm", _ptr(h), _ptr(table), _i32(_dt(table)), _ptr(ids), _f32_vec(weight, W, "the norm's weight"), _i64(T),
+          _i64(W), _i64(table.shape[0]), _i32(S), _f32(scale), _f32(eps), _stream())
+
+
+MAX_STREAMS = 32
+
+
+def stream_norm(h: torch.Tensor, y: Optional[torch.Tensor], mix: Optional[torch.Tensor], gain: Optional[torch.Tensor],
+                enter: Optional[torch.Tensor], weight: torch.Tensor, out: torch.Tensor, eps: float,
+                rows: Optional[torch.Tensor] = None) -> None:
+    """From one sublayer to the next over a stream of several copies, h float32 [T, S, W]:
+
+        x_j <- sum_i mix[i, j] x_i + gain[j] y   (with y only);   out = rmsnorm(sum_j enter[j] x_j) * weight
+
+    `mix` float32 [S, S] indexed [from, to], `gain`, `enter` float32 [S] (no `enter`: the plain sum), weight float32
+    [W], y and out of the run's type.  With `rows`, out[r] comes from row rows[r] and h stays as it was."""
+    T, S, W = h.shape
+    _need(h.dtype == torch.float32 and 1 <= S <= MAX_STREAMS, "the stream must be float32 [T, 1 .. 32, W]")
+    _need(weight.dtype == torch.float32 and weight.numel() == W and out.dim() == 2 and out.shape[1] == W, "width mismatch")
+    _need(y is None or (y.shape == (T, W) and y.dtype == out.dtype), "y must be [T, W] of out's type")
+    _need(y is None or (mix is not None and gain is not None), "a result that comes back needs the mix and its gains")
+    n_out = out.shape[0]
+    if rows is None:
+        _need(n_out == T, "out must have a row per row of h")
+    else:
+        _is_i32(rows, n_out)
+    fn = _functions.get("ix_stream_norm_needs_work")
+    if fn is None:
+        fn = _functions["ix_stream_norm_needs_work"] = lib().ix_stream_norm_needs_work
+    work = torch.empty((n_out, W), dtype=torch.float32, device=h.device) if fn(S, W) else None
+    _call("ix_stream_norm", _ptr(h), _ptr(y), _f32_vec(mix, S * S, "the mix"), _f32_vec(gain, S, "the gains"),
+          _f32_vec(enter, S, "the entering weights"), _ptr(weight), _ptr(out), _i32(_dt(out)), _ptr(rows), _ptr(work),
+          _i64(n_out), _i32(S), _i64(W), _f32(eps), _stream())
 
 
 # ---- attention over a compressed cache ------------------------------------------------------------------------------

@@ -12,8 +12,8 @@ element that the heads share, before they are rotated), `sink` (a learned number
 the softmax's denominator: no key, no value, not scaled, counted once), `value_dim` (values of another size than
 keys) and `value_position` (a position encoding over ALL of a value head: the value of position j is cached rotated
 by j, and every head's weighted sum at position i is rotated back by i, so that what a query receives depends on
-i - j only).  With any of these the step after the product is `ops.qkv_norm_rope_append`; with a sink, rotated values
-or values of another size the attention itself is the plain kernel.
+i - j only).  With any of these the step after the product is `ops.qkv_norm_rope_append`; with values of another size
+the attention itself is the plain kernel.  `softcap` c > 0: a score becomes c tanh(score / c) before the softmax.
 """
 from __future__ import annotations
 
@@ -35,7 +35,7 @@ class PagedAttention(Mixer):
                  out_bias: bool = False, window: int = 0, scale: Optional[float] = None,
                  position: Optional[PartSpec] = None, init_std: float = 0.02, value_dim: Optional[int] = None,
                  qk_norm: bool = False, qk_norm_eps: float = 1e-6, sink: bool = False,
-                 value_position: Optional[PartSpec] = None):
+                 value_position: Optional[PartSpec] = None, softcap: float = 0.0):
         if num_heads % num_kv_heads:
             raise ValueError(f"num_heads {num_heads} is not a multiple of num_kv_heads {num_kv_heads}")
         general = qk_norm or value_position is not None or (value_dim is not None and int(value_dim) != int(head_dim))
@@ -45,7 +45,9 @@ class PagedAttention(Mixer):
         self.hidden_size, self.num_heads, self.num_kv_heads = int(hidden_size), int(num_heads), int(num_kv_heads)
         self.head_dim, self.qkv_bias, self.window = int(head_dim), bool(qkv_bias), int(window)
         self.scale = float(scale) if scale is not None else self.head_dim ** -0.5
-        self.init_std = float(init_std)
+        self.init_std, self.softcap = float(init_std), float(softcap)
+        if self.softcap < 0:
+            raise ValueError("softcap must not be negative")
         self.position = build_part("position", position) if position is not None else None
         # the part of every head that the position encoding rotates: (first element, number of elements)
         self.rotated = (0, self.head_dim)
@@ -160,22 +162,25 @@ class PagedAttention(Mixer):
             ops.add_bias(y, self.b_out)
         return y
 
-    def attend(self, ctx, q, cache, out, turn_back=None) -> None:
+    def attend(self, ctx, q, cache, out, turn_back=None, gate=None) -> None:
         """bfloat16 with pages and heads in multiples of 16: the matrix-core kernels (the one that shares keys through
         LDS for the prompt portions of a step, the wavefront-level one for requests that bring few tokens and for
         steps of one token per request); else the plain one, which also knows a sink, values of another size than
-        keys and a result that is rotated back (`turn_back`: the table of the query's angles)."""
+        keys and a result that is rotated back (`turn_back`: the table of the query's angles).  `gate`:
+        rows [T, heads * value_dim] whose sigmoid multiplies the result."""
         page_size = cache.k.shape[2]
-        # a sink and a result that is rotated back: the wavefront-level matrix-core kernel knows both (the latter for
-        # heads of a multiple of 32); values of another size than keys: the plain kernel
-        special = self.sink is not None or turn_back is not None
+        # a sink, capped scores, a gate and a result that is rotated back: the wavefront-level matrix-core kernel knows all
+        # of them (the last for heads of a multiple of 32), the LDS-sharing one with tiles of 128 queries all but the
+        # last; values of another size than keys: the plain kernel
+        special = self.sink is not None or turn_back is not None or self.softcap > 0 or gate is not None
         fits = self.value_dim == self.head_dim and (turn_back is None or self.head_dim % 32 == 0)
         if q.dtype == torch.bfloat16 and page_size % 16 == 0 and self.head_dim % 16 == 0 and fits:
             T = ctx.num_tokens
-            more = {"sink": self.sink, "turn_back": turn_back} if special else {}
+            more = {"sink": self.sink, "turn_back": turn_back, "softcap": self.softcap, "gate": gate} if special else {}
             if not ctx.one_token_each:  # some request brings more than one token: the step's plan says who goes where
-                lds_fits = self.head_dim <= 128 and page_size & (page_size - 1) == 0 and not special
                 tile = WIDE_PREFILL_TILE if self.head_dim % 32 == 0 else PREFILL_TILE
+                lds_fits = (self.head_dim <= 128 and page_size & (page_size - 1) == 0
+                            and (not special or (turn_back is None and tile == WIDE_PREFILL_TILE)))
                 lds, waves = mixed_step_plan(ctx, self.window, self.num_heads, self.num_kv_heads, lds_fits, tile)
                 table = ctx.block_tables[cache.group]
                 if lds is not None:
@@ -183,14 +188,17 @@ class PagedAttention(Mixer):
                     work = None
                     if slices > 1:
                         work = ctx.rt.empty((T * self.num_heads * slices * (self.head_dim + 2),), torch.float32)
+                    shared = {"sink": self.sink, "softcap": self.softcap, "gate": gate} if special else {}
                     ops.attention_prefill(q, cache.k, cache.v, table, tiles, ctx.positions, out, self.scale,
-                                          self.window, tile, pairs, slices, work)
+                                          self.window, tile, pairs, slices, work, **shared)
                 for rows, tiles, positions, n_splits, grouped in waves:
                     # a launch that serves some of the step's requests gets their rows put side by side
                     qs = q if rows is None else q.index_select(0, rows)
                     outs = out if rows is None else torch.empty_like(qs)
                     if turn_back is not None:
                         more["turn_back"] = turn_back if rows is None else turn_back.index_select(0, rows)
+                    if gate is not None:
+                        more["gate"] = gate if rows is None else gate.index_select(0, rows)
                     work = None
                     if n_splits > 1:
                         work = ctx.rt.empty((qs.shape[0] * self.num_heads * n_splits * (self.head_dim + 2),),
@@ -209,7 +217,9 @@ class PagedAttention(Mixer):
                                n_splits, work, self.scale, self.window, tile, prefetch=True, grouped=grouped, **more)
         else:
             ops.attention_plain(q, cache.k, cache.v, ctx.block_tables[cache.group], ctx.seq_of_token, ctx.positions,
-                                out, self.scale, self.window, self.sink, turn_back)
+                                out, self.scale, self.window, self.sink, turn_back, self.softcap)
+            if gate is not None:
+                ops.sigmoid_gate(out.view(out.shape[0], -1), gate)
 
 
 # ---- the wavefront-level kernel (ops.attention_mfma)

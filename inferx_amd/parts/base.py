@@ -3,7 +3,7 @@
 A part is built from the parameters in its `PartSpec`, never from a config
 object, and does not know which model it is in.  Seven kinds:
 
-  Embedding         forward(ctx) -> the residual stream h, float32 [T, hidden]
+  Embedding         forward(ctx) -> the residual stream h, float32 [T, hidden] (or [T, copies, hidden])
   Norm              forward(ctx, h, delta=None, rows=None) -> normed activations
   PositionEncoding  prepare(ctx) -> whatever its mixer's kernels need this step
   Mixer             forward(ctx, x, cache) -> delta   (attention here)
@@ -12,6 +12,8 @@ object, and does not know which model it is in.  Seven kinds:
   Head              forward(ctx, x) -> float32 logits [rows, vocab]
   BranchGain        apply(delta) -> the delta with a learned gain per channel, applied where it is added
   TokenShift        forward(ctx, x, cache) -> rows blended with the rows of the tokens before them
+
+and the three tensors around a sublayer of a stream that is kept in several copies (kind "streams", see streams.py).
 
 Every part lists the tensors it needs (`param_specs`) under local names; the
 `PartSpec` maps those to checkpoint names.  `bind` receives the loaded tensors
@@ -267,13 +269,13 @@ class Block:
 
 _REGISTRIES: Dict[str, Dict[str, Callable[..., Any]]] = {
     "norm": {}, "position": {}, "mixer": {}, "feed_forward": {}, "block": {}, "embedding": {}, "head": {},
-    "gain": {}, "shift": {},
+    "gain": {}, "shift": {}, "streams": {},
 }
 
 
 def register_part(kind: str, name: str, factory: Callable[..., Any]) -> None:
-    """kind: 'norm' | 'position' | 'mixer' | 'feed_forward' | 'block' | 'embedding' | 'head' | 'gain' | 'shift'.  A block is
-    registered by its class (see `Block`), every other kind by a callable that takes the `PartSpec`'s parameters."""
+    """kind: 'norm' | 'position' | 'mixer' | 'feed_forward' | 'block' | 'embedding' | 'head' | 'gain' | 'shift' |
+    'streams'.  A block is registered by its class (see `Block`), every other kind by a callable that takes the `PartSpec`'s parameters."""
     if kind not in _REGISTRIES:
         raise KeyError(f"no such kind of part: {kind!r} (known: {', '.join(_REGISTRIES)})")
     _REGISTRIES[kind][name] = factory

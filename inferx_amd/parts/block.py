@@ -16,6 +16,7 @@ from .base import Block, LazyDelta, LazyNorm, register_part, resolve_delta
 from .dense_mlp import BiasedDelta
 from .gain_shift import WeightedSum
 from .norm import NormedDelta
+from .streams import StreamDelta
 
 
 class PreNormBlock(Block):
@@ -202,7 +203,38 @@ class PreNormBranchesBlock(Block):
         return self.feed_forward.forward(ctx, self.feed_forward_norm.forward(ctx, h, a))
 
 
+class HyperPreNormBlock(Block):
+    """`prenorm` over a stream of several copies: every sublayer reads a weighted sum of the copies and its result comes
+    back into a mix of them (see streams.py).
+
+        x = norm1(enter1(streams));  y = mixer(x);  streams = leave1(streams, y);  likewise with feed_forward
+
+    The feed-forward, its norm and its tensors may be left out together.  The last result stays pending."""
+
+    graph_safe = True
+    part_kinds = {"mixer": "mixer", "feed_forward": "feed_forward", "mixer_norm": "norm", "feed_forward_norm": "norm",
+                  "mixer_streams": "streams", "feed_forward_streams": "streams"}
+    optional_parts = ("feed_forward", "feed_forward_norm", "feed_forward_streams")
+
+    def __init__(self, parts):
+        super().__init__(parts)
+        present = [p is not None for p in (self.feed_forward, self.feed_forward_norm, self.feed_forward_streams)]
+        if any(present) != all(present):
+            raise KeyError("a feed-forward, the norm before it and its streams' tensors come together or not at all")
+
+    def forward(self, ctx, h, pending, caches):
+        if pending is None:
+            pending = StreamDelta(None, None)
+        x = self.mixer_norm.forward(ctx, h, pending.then(self.mixer_streams))
+        pending = StreamDelta(self.mixer.forward(ctx, x, caches.get("mixer")), self.mixer_streams)
+        if self.feed_forward is None:
+            return pending
+        x = self.feed_forward_norm.forward(ctx, h, pending.then(self.feed_forward_streams))
+        return StreamDelta(self.feed_forward.forward(ctx, x), self.feed_forward_streams)
+
+
 register_part("block", "prenorm", PreNormBlock)
+register_part("block", "hyper_prenorm", HyperPreNormBlock)
 register_part("block", "prenorm_branches", PreNormBranchesBlock)
 register_part("block", "parallel", ParallelBlock)
 register_part("block", "sandwich_norm", SandwichNormBlock)

@@ -16,20 +16,28 @@ from .base import LazyDelta, Norm, ParamSpec, register_part
 class RMSNorm(Norm):
     graph_safe = True
 
-    def __init__(self, width: int, eps: float, scalar: bool = False, groups: int = 1):
+    def __init__(self, width: int, eps: float, scalar: bool = False, groups: int = 1,
+                 offset: float = 0.0):
         """`scalar`: the weight is ONE number for all coordinates (a tensor without dimensions), spread over the
         width when it is bound, so that every kernel that applies an RMS norm takes it as it is.  `groups`: the
-        width is cut into that many equal consecutive runs, and each is divided by its own root mean square."""
+        width is cut into that many equal consecutive runs, and each is divided by its own root mean square.  `offset`:
+        what is added to the stored weight when it is bound (1 for weights that are stored around zero)."""
         self.width, self.eps, self.scalar, self.groups = int(width), float(eps), bool(scalar), int(groups)
         if self.groups < 1 or self.width % self.groups:
             raise ValueError(f"{groups} groups do not divide a width of {width}")
+        self.offset = float(offset)
         self.weight = None
 
     def param_specs(self) -> List[ParamSpec]:
-        return [ParamSpec("weight", () if self.scalar else (self.width,), init="ones")]
+        shape = () if self.scalar else (self.width,)
+        if self.offset:  # stored around zero, give or take what makes the whole about one
+            return [ParamSpec("weight", shape, std=0.1, mean=1.0 - self.offset)]
+        return [ParamSpec("weight", shape, init="ones")]
 
     def bind(self, tensors, rt) -> None:
         w = tensors["weight"]
+        if self.offset:
+            w = w.to(torch.float32) + self.offset
         self.weight = w.reshape(1).expand(self.width).contiguous() if self.scalar else w.contiguous()
 
     def rms_operands(self):

@@ -46,8 +46,10 @@ class ShortConv:
         self.weight = stack_rows([tensors[f"{n}.conv"] for n in names])
         self.weight_t = self.weight.to(torch.float32).t().contiguous()  # [taps, channels], for the kernel's 16-byte form
 
-    def apply(self, ctx, x, state, out_q, out_k, out_v, slots=None, cos_sin=None, silu: bool = False) -> None:
+    def apply(self, ctx, x, state, out_q, out_k, out_v, slots=None, cos_sin=None, silu: bool = False,
+              temperature=None) -> None:
         """`state`: the float32 view [slots, >= state_floats] of the requests' last inputs (see `ops.short_conv`)."""
         rows = ops.StepRows(ctx.seq_of_token, ctx.q_start, ctx.state_slots)
         ops.short_conv(x, self.bias, self.weight, state, rows, self.sizes, out_q, out_k, out_v, slots=slots,
-                       cos_sin=cos_sin, silu=silu, weight_t=self.weight_t, bias_f32=self.bias_f32)
+                       cos_sin=cos_sin, silu=silu, weight_t=self.weight_t, bias_f32=self.bias_f32,
+                       temperature=temperature)
