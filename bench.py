@@ -36,6 +36,7 @@ feed-forward width, vocabulary and layers), both through the step function, at a
     python bench.py --workload dezudra [--sizes 1k,2k] [--layers L] [--batch B] [--prompt-len C] [--prefill-tokens N]
     python bench.py --workload bibevik [--sizes 1k,2k] [--only bibevik|dezudra]       # Bibevik beside Dezudra
     python bench.py --workload gosuvik [--sizes 1k,2k] [--only gosuvik|dezudra]       # Gosuvik beside Dezudra
+    python bench.py --workload setopel [--sizes 1k,2k] [--only setopel|like_layers]   # Setopel beside other designs' like layers
 
 and a whole batch through the engine's loop (scheduler, portions, decode graphs as they come, sampling) at the same
 shape:
@@ -721,6 +722,94 @@ def run_gosuvik(args) -> int:
     return 0
 
 
+# Layer sizes for `--workload setopel`: width, query heads and key/value heads of `dim` numbers (retention: `heads` heads
+# of dim x dim; latent attention: `heads` heads over a latent of `rank`), copies of the stream, feed-forward width,
+# vocabulary
+SETOPEL_SIZES = {
+    "1k": dict(width=1024, heads=8, kv_heads=2, dim=128, rank=512, streams=4, ff=2816, vocab=32000),
+    "2k": dict(width=2048, heads=16, kv_heads=4, dim=128, rank=512, streams=4, ff=5632, vocab=32000),
+    "4k": dict(width=4096, heads=32, kv_heads=8, dim=128, rank=512, streams=4, ff=11008, vocab=32000),
+}
+
+
+def run_setopel(args) -> int:
+    """Prefill of one prompt and decode steps of a batch, through the step function, for the Setopel design (layers in
+    turn: attention, retention, latent attention, attention over the first layer's keys; four copies of the stream,
+    dense feed-forwards) and for a model put together from the like layers of the other designs in the same order and at
+    equal sizes (one stream, plain RMS norms: the Qwen2-MoE architecture's dense layers, Bibevik's lightning attention and
+    latent attention with 64 rotated numbers, the same feed-forwards).  One JSON line; per size and model milliseconds
+    and tokens a second of both phases, and Setopel's time over the other's."""
+    import torch
+    from inferx_amd.config import LayerSpec, ModelSpec, PartSpec, ScheduleEntry, config_from_dict, linear_head, token_embedding
+    from inferx_amd.engine.runtime import Runtime
+
+    L = args.layers or 4
+    B, C, N = args.batch, args.prompt_len, args.prefill_tokens
+    rt = Runtime(args.dtype, "cuda:0")
+    gen = torch.Generator().manual_seed(1234)
+    out = {}
+
+    def specs(z):
+        W, H, G, D, R, ff = z["width"], z["heads"], z["kv_heads"], z["dim"], z["rank"], z["ff"]
+        decay = [1.0 - 2.0 ** (-5 - 3 * h / H) for h in range(H)]
+        mlp = {"kind": "dense", "ff": ff}
+        attention = {"heads": H, "kv_heads": G, "dim": D, "vdim": D, "scale": D ** -0.5, "softcap": 50.0, "conv": 4,
+                     "q_temp": {"coef": 0.1, "every": 1024}}
+        order = [{"type": "attention", "mixer": attention, "mlp": mlp},
+                 {"type": "retention", "mixer": {"heads": H, "dim": D, "vdim": D, "decay": decay,
+                                                 "rot": {"dims": D, "base": 10000.0}}, "mlp": mlp},
+                 {"type": "latent_attention", "mixer": {"heads": H, "dim": D, "vdim": D, "kv_rank": R, "scale": D ** -0.5},
+                  "mlp": mlp},
+                 {"type": "attention", "mixer": dict(attention, kv_from=0), "mlp": mlp}]
+        mine = {"architecture": "Setopel", "vocab": z["vocab"], "width": W, "norm": {"eps": 1e-6}, "residual_mult": 0.5,
+                "streams": z["streams"], "layers": [order[i % 4] for i in range(L)]}
+        norm = PartSpec("rmsnorm", {"width": W, "eps": 1e-6})
+        named = lambda name: PartSpec("rmsnorm", {"width": W, "eps": 1e-6}, rename={"weight": name})
+        rope = lambda dims: PartSpec("rope", {"theta": 10000.0, "rotary_dim": dims})
+        mixers = [PartSpec("attention", {"hidden_size": W, "num_heads": H, "num_kv_heads": G, "head_dim": D, "position": rope(D)}),
+                  PartSpec("lightning_attention", {"hidden_size": W, "num_heads": H, "head_dim": D, "value_dim": D, "decay": decay}),
+                  PartSpec("latent_attention", {"hidden_size": W, "num_heads": H, "head_dim": D, "rot_dim": 64, "value_dim": D,
+                                                "kv_rank": R, "position": rope(64)})]
+        layers = []
+        for i in range(L):
+            at = lambda part, under: PartSpec(part.kind, part.params, prefix=f"l{i}.{under}.")
+            layers.append(LayerSpec("prenorm", {
+                "mixer_norm": at(norm, "n1"), "mixer": at(mixers[[0, 1, 2, 0][i % 4]], "mix"), "feed_forward_norm": at(norm, "n2"),
+                "feed_forward": PartSpec("dense_mlp", {"hidden_size": W, "width": ff}, prefix=f"l{i}.mlp.")}))
+        like = ModelSpec(architecture="like layers", hidden_size=W, vocab_size=z["vocab"], max_positions=0, layers=layers,
+                         schedule=[ScheduleEntry(i) for i in range(L)], embedding=token_embedding("embed", z["vocab"], W),
+                         final_norm=named("final.norm"), head=linear_head("head", z["vocab"], W))
+        return {"setopel": config_from_dict(mine).model_spec(), "like_layers": like}
+
+    for name in [n for n in args.sizes.split(",") if n]:
+        z = SETOPEL_SIZES[name]
+        res = {}
+        for which, spec in specs(z).items():
+            if args.only and which != args.only:
+                continue
+            log(f"{name}: {which}")
+            pre, dec = _time_prefill_and_decode(args, rt, spec, z["vocab"], gen)
+            res[which] = {"prefill_ms": round(pre * 1e3, 3), "prefill_tokens_s": round(N / pre, 1),
+                          "decode_ms": round(dec * 1e3, 3), "decode_tokens_s": round(B / dec, 1)}
+            log(f"{name}: {which}: {res[which]}")
+        if len(res) == 2:
+            res["setopel_over_like_layers"] = {
+                "prefill": round(res["setopel"]["prefill_ms"] / res["like_layers"]["prefill_ms"], 3),
+                "decode": round(res["setopel"]["decode_ms"] / res["like_layers"]["decode_ms"], 3)}
+        out[name] = dict(res, sizes=z)
+    first = out[next(iter(out))]
+    mine = first.get("setopel") or next(iter(v for v in first.values() if isinstance(v, dict) and "decode_ms" in v))
+    print(json.dumps({
+        "metric": f"Setopel decode tok/s @ batch {B} ({C}-token contexts), first size", "value": mine["decode_tokens_s"],
+        "unit": "tokens/s", "n_gpus": 1, "steps": args.steps, "warmup": args.warmup,
+        "ms_per_step": mine["decode_ms"], "higher_is_better": True, "scaling": "weak", "vs_baseline": None,
+        "dtype": "bf16" if args.dtype == "bfloat16" else "fp32", "data": "synthetic: seeded random weights and token ids",
+        "config": {"model": "Setopel beside the like layers of other designs at equal sizes", "layers": L, "global_batch": B,
+                   "seq_len": C, "prefill_tokens": N, "parallelism": "single GPU", "page_size": PAGE},
+        "sizes": out}), flush=True)
+    return 0
+
+
 def run_pelalix(args) -> int:
     """Prefill of one prompt and decode steps of a batch, through the step function, for the Pelalix design and for
     the Qwen2-MoE architecture's dense layers (attention with rotation, RMS norms, the same gated feed-forward) at
@@ -804,7 +893,7 @@ def main() -> int:
     ap.add_argument("--scarce", action="store_true", help="offline: so few pages that sequences are preempted")
     ap.add_argument("--workload", default="decode",
                     choices=["decode", "mixed", "long", "mixed-small", "offline", "portion", "pelalix", "dezudra", "bibevik",
-                             "gosuvik"],
+                             "gosuvik", "setopel"],
                     help="decode, mixed-small: the Qwen1.5-MoE-A2.7B shape (decode is the default); mixed, long: the "
                          "Qwen2-57B-A14B shape")
     ap.add_argument("--batch", type=int, default=8)
@@ -816,8 +905,8 @@ def main() -> int:
     ap.add_argument("--prefill-context", type=int, default=0,
                     help="portion: tokens that the request has read before the timed portion")
     ap.add_argument("--shape", default="a27b", choices=["a27b", "57b"], help="portion: whose layer sizes")
-    ap.add_argument("--sizes", default="2k,4k", help="pelalix, dezudra, bibevik, gosuvik: which of the layer sizes " + ", ".join(PELALIX_SIZES))
-    ap.add_argument("--only", default="", help="bibevik, gosuvik: time one of the two models only (by its name)")
+    ap.add_argument("--sizes", default="2k,4k", help="pelalix, dezudra, bibevik, gosuvik, setopel: which of the layer sizes " + ", ".join(PELALIX_SIZES))
+    ap.add_argument("--only", default="", help="bibevik, gosuvik, setopel: time one of the two models only (by its name)")
     ap.add_argument("--prompt-len", type=int, default=PROMPT,
                     help="tokens of every request's prompt before it decodes (the context of the decode steps)")
     args = ap.parse_args()
@@ -825,9 +914,9 @@ def main() -> int:
         print("bench.py: this engine runs on one GPU; --gpus N > 1 is not supported")
         return 2
     if args.steps is None:
-        args.steps = {"decode": 32, "mixed": 8, "long": 256, "mixed-small": 24, "offline": 0, "portion": 2, "pelalix": 32, "dezudra": 32, "bibevik": 32, "gosuvik": 32}[args.workload]
+        args.steps = {"decode": 32, "mixed": 8, "long": 256, "mixed-small": 24, "offline": 0, "portion": 2, "pelalix": 32, "dezudra": 32, "bibevik": 32, "gosuvik": 32, "setopel": 32}[args.workload]
     if args.warmup is None:
-        args.warmup = {"decode": 4, "mixed": 2, "long": 4, "mixed-small": 4, "offline": 0, "portion": 1, "pelalix": 4, "dezudra": 4, "bibevik": 4, "gosuvik": 4}[args.workload]
+        args.warmup = {"decode": 4, "mixed": 2, "long": 4, "mixed-small": 4, "offline": 0, "portion": 1, "pelalix": 4, "dezudra": 4, "bibevik": 4, "gosuvik": 4, "setopel": 4}[args.workload]
     if args.workload == "offline":
         return run_offline(args)
     if args.workload == "portion":
@@ -840,6 +929,8 @@ def main() -> int:
         return run_bibevik(args)
     if args.workload == "gosuvik":
         return run_gosuvik(args)
+    if args.workload == "setopel":
+        return run_setopel(args)
     if args.workload != "decode":
         return run_57b(args)
     if args.layers is None:

@@ -32,7 +32,7 @@ struct LinearChunks {
   const float* w_head;            // [heads]
   const float2* cos_sin;          // [T, half] or null
   float k_scale;
-  int half, silu, heads, dim, vdim, vec;
+  int half, silu, heads, dim, vdim;
   const int32_t* chunk_row0;      // [chunks] first row in the step
   const int32_t* chunk_rows;      // [chunks] 1 .. 64
   float* kv;                      // [chunks, heads, vdim, dim]: a chunk's outer products, then the state before it
@@ -42,47 +42,90 @@ struct LinearChunks {
 __device__ __forceinline__ float lc_power(float lg, int n) { return n == 0 ? 1.0f : exp2f(static_cast<float>(n) * lg); }
 __device__ __forceinline__ float lc_silu(float x) { return x / (1.0f + expf(-x)); }
 
-__device__ __forceinline__ float4 lc_load4(const float* p) { return *reinterpret_cast<const float4*>(p); }
-__device__ __forceinline__ float4 lc_load4(const bf16_t* p) {
-  const uint2 d = *reinterpret_cast<const uint2*>(p);
-  return float4{__uint_as_float(d.x << 16), __uint_as_float(d.x & 0xffff0000u), __uint_as_float(d.y << 16),
-                __uint_as_float(d.y & 0xffff0000u)};
+// four consecutive numbers as they come from memory, opened into floats when they are used
+template <typename T> struct lc_piece;
+template <> struct lc_piece<float> { float4 a; };
+template <> struct lc_piece<bf16_t> { uint2 a; };
+__device__ __forceinline__ float4 lc_open(const lc_piece<float>& p) { return p.a; }
+__device__ __forceinline__ float4 lc_open(const lc_piece<bf16_t>& p) {
+  return float4{__uint_as_float(p.a.x << 16), __uint_as_float(p.a.x & 0xffff0000u), __uint_as_float(p.a.y << 16),
+                __uint_as_float(p.a.y & 0xffff0000u)};
 }
-
-// four numbers of a head's row from d on (zeros past its `n` numbers); vec: the row lies on boundaries of four numbers
-template <typename T>
-__device__ __forceinline__ float4 lc_take4(const T* row, int d, int n, int vec) {
-  if (vec) return lc_load4(row + d);
-  float4 x;
-  x.x = ix_load(row + d);
-  x.y = d + 1 < n ? ix_load(row + d + 1) : 0.f;
-  x.z = d + 2 < n ? ix_load(row + d + 2) : 0.f;
-  x.w = d + 3 < n ? ix_load(row + d + 3) : 0.f;
-  return x;
-}
-
-// a head's row piece as it enters the products: silu, rotation
-template <typename T>
-__device__ __forceinline__ float4 lc_operand4(const LinearChunks& a, const T* row, int64_t t, int d) {
-  float4 x = lc_take4(row, d, a.dim, a.vec);
-  if (a.silu) return float4{lc_silu(x.x), lc_silu(x.y), lc_silu(x.z), lc_silu(x.w)};
-  if (a.cos_sin && d < 2 * a.half) {
-    float y[4] = {x.x, x.y, x.z, x.w};
-#pragma unroll
-    for (int e = 0; e < 4; ++e) {
-      const int i = d + e;
-      if (i >= 2 * a.half) continue;
-      const bool low = i < a.half;
-      const float2 c = a.cos_sin[t * a.half + (low ? i : i - a.half)];
-      const float other = ix_load(row + (low ? i + a.half : i - a.half));
-      y[e] = low ? y[e] * c.x - other * c.y : y[e] * c.x + other * c.y;
-    }
-    x = float4{y[0], y[1], y[2], y[3]};
+// four numbers of a row from d on (zeros past its `n` numbers; d < n).  VEC: the row lies on boundaries of four numbers
+template <bool VEC>
+__device__ __forceinline__ lc_piece<float> lc_ask(const float* row, int d, int n) {
+  lc_piece<float> p;
+  if constexpr (VEC) {
+    p.a = *reinterpret_cast<const float4*>(row + d);
+  } else {
+    p.a = float4{row[d], d + 1 < n ? row[d + 1] : 0.f, d + 2 < n ? row[d + 2] : 0.f, d + 3 < n ? row[d + 3] : 0.f};
   }
-  return x;
+  return p;
+}
+template <bool VEC>
+__device__ __forceinline__ lc_piece<bf16_t> lc_ask(const bf16_t* row, int d, int n) {
+  lc_piece<bf16_t> p;
+  if constexpr (VEC) {
+    p.a = *reinterpret_cast<const uint2*>(row + d);
+  } else {
+    const uint32_t e1 = d + 1 < n ? row[d + 1].bits : 0, e2 = d + 2 < n ? row[d + 2].bits : 0, e3 = d + 3 < n ? row[d + 3].bits : 0;
+    p.a = uint2{row[d].bits | e1 << 16, e2 | e3 << 16};
+  }
+  return p;
+}
+__device__ __forceinline__ float4 lc_silu4(float4 x) { return float4{lc_silu(x.x), lc_silu(x.y), lc_silu(x.z), lc_silu(x.w)}; }
+__device__ __forceinline__ float4 lc_scaled(float4 x, float f) { return float4{x.x * f, x.y * f, x.z * f, x.w * f}; }
+
+// A tile of LC_ROWS rows of W numbers, LC_THREADS threads, four numbers each and turn: piece `u` of this thread.  Every
+// piece of a tile is asked for before the first is used (rows past the chunk's last repeat it, numbers past the row's
+// end repeat its first four; both are made zero on the way into LDS).
+template <int W>
+struct LcTile {
+  static constexpr int PER = LC_ROWS * (W / 4) / LC_THREADS;
+  static __device__ __forceinline__ int row(int u) { return (u * LC_THREADS + static_cast<int>(threadIdx.x)) / (W / 4); }
+  static __device__ __forceinline__ int d(int u) { return 4 * ((u * LC_THREADS + static_cast<int>(threadIdx.x)) % (W / 4)); }
+};
+
+// piece u of a head's rows (of `n` numbers), and the piece it is rotated with
+template <typename T, int W, bool VEC>
+__device__ __forceinline__ void lc_ask_tile(const T* src, int64_t stride, int64_t row0, int rows, int n,
+                                            lc_piece<T> (&p)[LcTile<W>::PER]) {
+#pragma unroll
+  for (int u = 0; u < LcTile<W>::PER; ++u) {
+    const int d = LcTile<W>::d(u);
+    p[u] = lc_ask<VEC>(src + (row0 + min(LcTile<W>::row(u), rows - 1)) * stride, d < n ? d : 0, n);
+  }
 }
 
-template <typename T, int DIM>
+// a piece as it enters the products: silu, or the rotation (its partners read from memory again: they are in the cache)
+template <typename T, bool VEC>
+__device__ __forceinline__ float4 lc_operand(const LinearChunks& a, const lc_piece<T>& p, const T* row, int64_t t, int d) {
+  float4 x = lc_open(p);
+  if (a.silu) return lc_silu4(x);
+  if (!a.cos_sin || d >= 2 * a.half) return x;
+  if (VEC && (a.half & 3) == 0) {  // four numbers of the lower half or of the upper, and four partners
+    const bool low = d < a.half;
+    const float4 o = lc_open(lc_ask<VEC>(row, low ? d + a.half : d - a.half, a.dim));
+    const float4* cs = reinterpret_cast<const float4*>(a.cos_sin + t * a.half + (low ? d : d - a.half));
+    const float4 c0 = cs[0], c1 = cs[1];  // (cos, sin) of four angles
+    const float sg = low ? -1.0f : 1.0f;
+    return float4{x.x * c0.x + o.x * (sg * c0.y), x.y * c0.z + o.y * (sg * c0.w), x.z * c1.x + o.z * (sg * c1.y),
+                  x.w * c1.z + o.w * (sg * c1.w)};
+  }
+  float y[4] = {x.x, x.y, x.z, x.w};
+#pragma unroll
+  for (int e = 0; e < 4; ++e) {
+    const int i = d + e;
+    if (i >= 2 * a.half) continue;
+    const bool low = i < a.half;
+    const float2 c = a.cos_sin[t * a.half + (low ? i : i - a.half)];
+    const float other = ix_load(row + (low ? i + a.half : i - a.half));
+    y[e] = low ? y[e] * c.x - other * c.y : y[e] * c.x + other * c.y;
+  }
+  return float4{y[0], y[1], y[2], y[3]};
+}
+
+template <typename T, int DIM, bool VEC>
 __global__ void __launch_bounds__(LC_THREADS) lc_outer_kernel(LinearChunks a) {
   __shared__ __attribute__((aligned(16))) float k_s[LC_ROWS * DIM];
   __shared__ __attribute__((aligned(16))) float v_s[LC_ROWS * LC_COLS];
@@ -95,28 +138,26 @@ __global__ void __launch_bounds__(LC_THREADS) lc_outer_kernel(LinearChunks a) {
   const T* v = static_cast<const T*>(a.v) + static_cast<int64_t>(head) * a.vdim + v0;
   const int cols = min(LC_COLS, a.vdim - v0);
   const int n2 = (n + 1) & ~1;  // (rows are taken in pairs)
-#pragma unroll 4
-  for (int id = tid; id < LC_ROWS * (DIM / 4); id += LC_THREADS) {
-    const int row = id / (DIM / 4), d = 4 * (id % (DIM / 4));
-    if (row >= n2) continue;
-    float4 x = float4{0.f, 0.f, 0.f, 0.f};
-    if (row < n && d < a.dim) {
-      x = lc_operand4(a, k + (row0 + row) * a.k_stride, row0 + row, d);
-      const float f = a.k_scale * lc_power(lg, n - 1 - row);
-      x = float4{x.x * f, x.y * f, x.z * f, x.w * f};
+  const float4 zero = float4{0.f, 0.f, 0.f, 0.f};
+  {
+    lc_piece<T> kp[LcTile<DIM>::PER], vp[LcTile<LC_COLS>::PER];
+    lc_ask_tile<T, DIM, VEC>(k, a.k_stride, row0, n, a.dim, kp);
+    lc_ask_tile<T, LC_COLS, VEC>(v, a.v_stride, row0, n, cols, vp);
+#pragma unroll
+    for (int u = 0; u < LcTile<DIM>::PER; ++u) {
+      const int row = LcTile<DIM>::row(u), d = LcTile<DIM>::d(u);
+      float4 x = zero;
+      if (row < n && d < a.dim)
+        x = lc_scaled(lc_operand<T, VEC>(a, kp[u], k + (row0 + row) * a.k_stride, row0 + row, d), a.k_scale * lc_power(lg, n - 1 - row));
+      *reinterpret_cast<float4*>(k_s + row * DIM + d) = x;
     }
-    *reinterpret_cast<float4*>(k_s + row * DIM + d) = x;
-  }
-#pragma unroll 4
-  for (int id = tid; id < LC_ROWS * (LC_COLS / 4); id += LC_THREADS) {
-    const int row = id / (LC_COLS / 4), d = 4 * (id % (LC_COLS / 4));
-    if (row >= n2) continue;
-    float4 x = float4{0.f, 0.f, 0.f, 0.f};
-    if (row < n && d < cols) {
-      x = lc_take4(v + (row0 + row) * a.v_stride, d, cols, a.vec);
-      if (a.silu) x = float4{lc_silu(x.x), lc_silu(x.y), lc_silu(x.z), lc_silu(x.w)};
+#pragma unroll
+    for (int u = 0; u < LcTile<LC_COLS>::PER; ++u) {
+      const int row = LcTile<LC_COLS>::row(u), d = LcTile<LC_COLS>::d(u);
+      float4 x = (row < n && d < cols) ? lc_open(vp[u]) : zero;
+      if (a.silu) x = lc_silu4(x);
+      *reinterpret_cast<float4*>(v_s + row * LC_COLS + d) = x;
     }
-    *reinterpret_cast<float4*>(v_s + row * LC_COLS + d) = x;
   }
   __syncthreads();
   if (32 * wave >= cols) return;
@@ -180,7 +221,7 @@ lc_chain_kernel(float* __restrict__ kv, const float* __restrict__ w_head, const 
   for (int e = 0; e < E; ++e) sp[e] = x[e];
 }
 
-template <typename T, int DIM>
+template <typename T, int DIM, bool VEC>
 __global__ void __launch_bounds__(LC_THREADS) lc_result_kernel(LinearChunks a) {
   constexpr int LD = DIM + 4;  // (rows of a tile read at one place then fall on different banks)
   __shared__ __attribute__((aligned(16))) float r_s[LC_ROWS * LD];
@@ -210,29 +251,30 @@ __global__ void __launch_bounds__(LC_THREADS) lc_result_kernel(LinearChunks a) {
   const T* r = static_cast<const T*>(a.r) + static_cast<int64_t>(head) * a.dim;
   const T* k = static_cast<const T*>(a.k) + static_cast<int64_t>(head) * a.dim;
   const T* v = static_cast<const T*>(a.v) + static_cast<int64_t>(head) * a.vdim + v0;
-  const int filled = two ? LC_ROWS : 32;
-#pragma unroll 4
-  for (int id = tid; id < LC_ROWS * (DIM / 4); id += LC_THREADS) {
-    const int row = id / (DIM / 4), d = 4 * (id % (DIM / 4));
-    if (row >= filled) continue;
-    float4 x = float4{0.f, 0.f, 0.f, 0.f}, y = x;
-    if (row < n && d < a.dim) {
-      x = lc_operand4(a, r + (row0 + row) * a.r_stride, row0 + row, d);
-      y = lc_operand4(a, k + (row0 + row) * a.k_stride, row0 + row, d);
+  {
+    const float4 zero = float4{0.f, 0.f, 0.f, 0.f};
+    lc_piece<T> rp[LcTile<DIM>::PER], kp[LcTile<DIM>::PER], vp[LcTile<LC_COLS>::PER];
+    lc_ask_tile<T, DIM, VEC>(r, a.r_stride, row0, n, a.dim, rp);
+    lc_ask_tile<T, DIM, VEC>(k, a.k_stride, row0, n, a.dim, kp);
+    lc_ask_tile<T, LC_COLS, VEC>(v, a.v_stride, row0, n, cols, vp);
+#pragma unroll
+    for (int u = 0; u < LcTile<DIM>::PER; ++u) {
+      const int row = LcTile<DIM>::row(u), d = LcTile<DIM>::d(u);
+      float4 x = zero, y = zero;
+      if (row < n && d < a.dim) {
+        x = lc_operand<T, VEC>(a, rp[u], r + (row0 + row) * a.r_stride, row0 + row, d);
+        y = lc_scaled(lc_operand<T, VEC>(a, kp[u], k + (row0 + row) * a.k_stride, row0 + row, d), a.k_scale);
+      }
+      *reinterpret_cast<float4*>(r_s + row * LD + d) = x;
+      *reinterpret_cast<float4*>(k_s + row * LD + d) = y;
     }
-    *reinterpret_cast<float4*>(r_s + row * LD + d) = x;
-    *reinterpret_cast<float4*>(k_s + row * LD + d) = float4{y.x * a.k_scale, y.y * a.k_scale, y.z * a.k_scale, y.w * a.k_scale};
-  }
-#pragma unroll 4
-  for (int id = tid; id < LC_ROWS * (LC_COLS / 4); id += LC_THREADS) {
-    const int row = id / (LC_COLS / 4), d = 4 * (id % (LC_COLS / 4));
-    if (row >= filled) continue;
-    float4 x = float4{0.f, 0.f, 0.f, 0.f};
-    if (row < n && d < cols) {
-      x = lc_take4(v + (row0 + row) * a.v_stride, d, cols, a.vec);
-      if (a.silu) x = float4{lc_silu(x.x), lc_silu(x.y), lc_silu(x.z), lc_silu(x.w)};
+#pragma unroll
+    for (int u = 0; u < LcTile<LC_COLS>::PER; ++u) {
+      const int row = LcTile<LC_COLS>::row(u), d = LcTile<LC_COLS>::d(u);
+      float4 x = (row < n && d < cols) ? lc_open(vp[u]) : zero;
+      if (a.silu) x = lc_silu4(x);
+      *reinterpret_cast<float4*>(v_s + row * LC_COLS + d) = x;
     }
-    *reinterpret_cast<float4*>(v_s + row * LC_COLS + d) = x;
   }
   __syncthreads();
   // ---- the weights w^(i - j) (r_i . k_j), j <= i: a tile of 32 x 32 per wavefront (the one above the diagonal is empty)
@@ -339,18 +381,23 @@ extern "C" int ix_linear_chunks(const void* r, const void* k, const void* v, int
   a.half = half; a.silu = silu; a.heads = heads; a.dim = dim; a.vdim = vdim;
   a.chunk_row0 = chunk_row0; a.chunk_rows = chunk_rows; a.kv = kv; a.out = out;
   const uintptr_t rows = reinterpret_cast<uintptr_t>(r) | reinterpret_cast<uintptr_t>(k) | reinterpret_cast<uintptr_t>(v);
-  a.vec = (rows & 15) == 0 && (r_stride | k_stride | v_stride) % 4 == 0 && vdim % 4 == 0;
+  const bool vec = (rows & 15) == 0 && (r_stride | k_stride | v_stride) % 4 == 0 && vdim % 4 == 0;
   dim3 grid(heads, chunks, (vdim + LC_COLS - 1) / LC_COLS), block(LC_THREADS);
   const int64_t per_head = static_cast<int64_t>(dim) * vdim;
   const bool fours = per_head % 4 == 0 && state_stride % 4 == 0 && (reinterpret_cast<uintptr_t>(state) & 15) == 0;
   const int64_t threads = fours ? per_head / 4 : per_head;
   dim3 chain(static_cast<unsigned>((threads + 255) / 256), heads, seqs);
-#define BY_DIM(KERNEL, T)                                                                            \
-  if (dim <= 32) hipLaunchKernelGGL((KERNEL<T, 32>), grid, block, 0, stream, a);                     \
-  else if (dim <= 64) hipLaunchKernelGGL((KERNEL<T, 64>), grid, block, 0, stream, a);                \
-  else if (dim <= 96) hipLaunchKernelGGL((KERNEL<T, 96>), grid, block, 0, stream, a);                \
-  else hipLaunchKernelGGL((KERNEL<T, 128>), grid, block, 0, stream, a)
-  if (dtype == IX_F32) { BY_DIM(lc_outer_kernel, float); } else { BY_DIM(lc_outer_kernel, bf16_t); }
+#define BY_DIM(KERNEL, T, VEC)                                                                       \
+  if (dim <= 32) hipLaunchKernelGGL((KERNEL<T, 32, VEC>), grid, block, 0, stream, a);                \
+  else if (dim <= 64) hipLaunchKernelGGL((KERNEL<T, 64, VEC>), grid, block, 0, stream, a);           \
+  else if (dim <= 96) hipLaunchKernelGGL((KERNEL<T, 96, VEC>), grid, block, 0, stream, a);           \
+  else hipLaunchKernelGGL((KERNEL<T, 128, VEC>), grid, block, 0, stream, a)
+#define BY_TYPE(KERNEL)                                     \
+  if (dtype == IX_F32 && vec) { BY_DIM(KERNEL, float, true); }   \
+  else if (dtype == IX_F32) { BY_DIM(KERNEL, float, false); }    \
+  else if (vec) { BY_DIM(KERNEL, bf16_t, true); }                \
+  else { BY_DIM(KERNEL, bf16_t, false); }
+  BY_TYPE(lc_outer_kernel)
   if (ix_check_launch("ix_linear_chunks: outer products")) return 1;
   if (fours)
     hipLaunchKernelGGL(lc_chain_kernel<4>, chain, dim3(256), 0, stream, kv, w_head, chunk_rows, seq_first, seq_count, seq_ids,
@@ -359,7 +406,8 @@ extern "C" int ix_linear_chunks(const void* r, const void* k, const void* v, int
     hipLaunchKernelGGL(lc_chain_kernel<1>, chain, dim3(256), 0, stream, kv, w_head, chunk_rows, seq_first, seq_count, seq_ids,
                        state_slots, state, state_stride, heads, per_head);
   if (ix_check_launch("ix_linear_chunks: chain")) return 1;
-  if (dtype == IX_F32) { BY_DIM(lc_result_kernel, float); } else { BY_DIM(lc_result_kernel, bf16_t); }
+  BY_TYPE(lc_result_kernel)
+#undef BY_TYPE
 #undef BY_DIM
   return ix_check_launch("ix_linear_chunks");
 }

@@ -378,16 +378,168 @@ __global__ void __launch_bounds__(CONV_THREADS) short_conv_vec8_kernel(ConvArgs 
   }
 }
 
+// The same for prompt portions without a rotation, at most four taps: a thread owns eight channels of sixteen
+// consecutive rows, so that taps, bias and every input are read once, and values that sixteen consecutive places of a
+// page take are written sixteen at a time.  A row whose inputs all lie in its own portion (its place i >= taps - 1) is
+// formed here; the portion's first rows, a last row that is among them, and the new state belong to one further
+// workgroup per request (blockIdx.x < requests), which alone reads and writes the state.
+#define CONV_TILE 16
+#define CONV_TILE_THREADS 128
+
+template <int TAPS>
+__global__ void __launch_bounds__(CONV_TILE_THREADS)
+short_conv_tile_kernel(ConvArgs a, const float* __restrict__ wt, const float* __restrict__ bias_f, int vunits,
+                       int requests, int tokens) {
+  __shared__ int32_t page_s[CONV_TILE], off_s[CONV_TILE], formed_s[CONV_TILE];
+  __shared__ float temp_s[CONV_TILE];
+  __shared__ int run_s;
+  const int unit = blockIdx.y * CONV_TILE_THREADS + threadIdx.x;
+  const bool live = unit < vunits;
+  const int c0 = 8 * (live ? unit : vunits - 1);
+  const uint16_t* in = static_cast<const uint16_t*>(a.in);
+  if (static_cast<int>(blockIdx.x) < requests) {  // (started first: a chain of reads, worked beside the tiles)
+    const int seq = blockIdx.x;
+    const int64_t row0 = a.q_start[seq];
+    const int n = a.q_start[seq + 1] - static_cast<int>(row0);
+    if (n <= 0 || !live) return;
+    float* st = a.state + static_cast<int64_t>(a.state_slots[seq]) * a.state_stride;
+    // everything that is needed is read at once: the state before, the portion's first inputs and its last ones
+    Conv8 u[2 * TAPS], tail[TAPS];
+#pragma unroll
+    for (int r = 0; r < TAPS - 1; ++r) {
+      u[r] = conv_input8(a, bias_f, in, st, row0, r - (TAPS - 1), c0);
+      u[TAPS - 1 + r] = conv_input8(a, bias_f, in, st, row0, min(r, n - 1), c0);
+      tail[r] = conv_input8(a, bias_f, in, st, row0, n - (TAPS - 1) + r, c0);
+    }
+#pragma unroll
+    for (int i = 0; i < TAPS - 1; ++i) {
+      if (i >= n) break;
+      Conv8 y;
+#pragma unroll
+      for (int e = 0; e < 8; ++e) y.x[e] = 0.f;
+#pragma unroll
+      for (int j = 0; j < TAPS; ++j)
+#pragma unroll
+        for (int e = 0; e < 8; ++e) y.x[e] += wt[static_cast<int64_t>(j) * a.channels + c0 + e] * u[i + j].x[e];
+      if (a.silu) {
+#pragma unroll
+        for (int e = 0; e < 8; ++e) y.x[e] = y.x[e] / (1.0f + expf(-y.x[e]));
+      }
+      const float temp = (a.temp_every > 0.f && c0 < a.q_channels) ? conv_temperature(a, row0 + i) : 1.0f;
+#pragma unroll
+      for (int e = 0; e < 8; ++e) y.x[e] *= temp;
+      conv_store8(a, row0 + i, c0, y);
+    }
+#pragma unroll
+    for (int r = 0; r < TAPS - 1; ++r) {
+      float* dst = st + static_cast<int64_t>(r) * a.channels + c0;
+      *reinterpret_cast<conv_f32x4*>(dst) = conv_f32x4{tail[r].x[0], tail[r].x[1], tail[r].x[2], tail[r].x[3]};
+      *reinterpret_cast<conv_f32x4*>(dst + 4) = conv_f32x4{tail[r].x[4], tail[r].x[5], tail[r].x[6], tail[r].x[7]};
+    }
+    return;
+  }
+  const int r0 = (static_cast<int>(blockIdx.x) - requests) * CONV_TILE;
+  conv_u32x4 raw[CONV_TILE + TAPS - 1];  // the inputs of rows r0 - (taps - 1) .. r0 + 15
+#pragma unroll
+  for (int i = 0; i < CONV_TILE + TAPS - 1; ++i)
+    raw[i] = *reinterpret_cast<const conv_u32x4*>(in + static_cast<int64_t>(min(max(r0 - (TAPS - 1) + i, 0), tokens - 1)) * a.in_stride + c0);
+  float w[TAPS][8], b[8];
+#pragma unroll
+  for (int j = 0; j < TAPS; ++j)
+#pragma unroll
+    for (int e = 0; e < 8; ++e) w[j][e] = wt[static_cast<int64_t>(j) * a.channels + c0 + e];
+#pragma unroll
+  for (int e = 0; e < 8; ++e) b[e] = bias_f ? bias_f[c0 + e] : 0.f;
+  // what the workgroup needs to know of its rows, a row per lane: whether it is formed here, its place in the cache, its
+  // temperature; and whether all sixteen places lie side by side on one page
+  if (threadIdx.x < CONV_TILE) {
+    const int i = threadIdx.x, row = min(r0 + i, tokens - 1);
+    const bool formed = r0 + i < tokens && row - a.q_start[a.seq_of_token[row]] >= TAPS - 1;
+    const int slot = a.slots ? a.slots[row] : 0, slot0 = a.slots ? a.slots[r0] : 0;
+    const int page = a.slots ? slot / a.page_size : 0, off = a.slots ? slot - page * a.page_size : 0;
+    formed_s[i] = formed;
+    page_s[i] = page;
+    off_s[i] = off;
+    temp_s[i] = a.temp_every > 0.f ? conv_temperature(a, row) : 1.0f;
+    const bool beside = a.slots && a.page_size % 8 == 0 && slot0 % 8 == 0 && formed && slot == slot0 + i &&
+                        off + CONV_TILE - i <= a.page_size && off >= i;
+    const uint64_t all = __ballot(beside);
+    if (i == 0) run_s = (all & 0xffffu) == 0xffffu;
+  }
+  __syncthreads();
+  if (!live) return;
+  const bool is_q = c0 < a.q_channels, is_v = c0 >= a.q_channels + a.k_channels;
+  const bool run = run_s != 0;
+  // where the thread's channels of a row go: plain rows, or the head's place in a page
+  const int cx = is_q ? c0 : (is_v ? c0 - a.q_channels - a.k_channels : c0 - a.q_channels);
+  const int dim = is_v ? a.value_dim : a.head_dim, heads = (is_v ? a.v_channels : a.k_channels) / dim;
+  const int head = cx / dim, e0 = cx % dim;
+  uint16_t* base = static_cast<uint16_t*>(is_q ? a.out_q : (is_v ? a.out_v : a.out_k));
+  const int64_t row_stride = is_q ? a.q_channels : (is_v ? a.v_channels : a.k_channels);
+  const bool paged = !is_q && a.slots;
+  conv_u32x4 vrows[CONV_TILE];
+#pragma unroll
+  for (int i = 0; i < CONV_TILE; ++i) {
+    Conv8 y;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) y.x[e] = 0.f;
+#pragma unroll
+    for (int j = 0; j < TAPS; ++j)
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        y.x[2 * e] += w[j][2 * e] * (__uint_as_float(raw[i + j][e] << 16) + b[2 * e]);
+        y.x[2 * e + 1] += w[j][2 * e + 1] * (__uint_as_float(raw[i + j][e] & 0xffff0000u) + b[2 * e + 1]);
+      }
+    if (a.silu) {
+#pragma unroll
+      for (int e = 0; e < 8; ++e) y.x[e] = y.x[e] / (1.0f + expf(-y.x[e]));
+    }
+    if (is_q) {
+      const float temp = temp_s[i];
+#pragma unroll
+      for (int e = 0; e < 8; ++e) y.x[e] *= temp;
+    }
+    vrows[i] = conv_pack8(y);
+    if (!formed_s[i] || (is_v && run)) continue;
+    if (!paged) {
+      *reinterpret_cast<conv_u32x4*>(base + static_cast<int64_t>(r0 + i) * row_stride + cx) = vrows[i];
+    } else if (!is_v) {
+      *reinterpret_cast<conv_u32x4*>(base + ((static_cast<int64_t>(page_s[i]) * heads + head) * a.page_size + off_s[i]) * dim + e0) = vrows[i];
+    } else {
+      uint16_t* dst = base + ((static_cast<int64_t>(page_s[i]) * heads + head) * dim + e0) * a.page_size + off_s[i];
+#pragma unroll
+      for (int e = 0; e < 8; ++e)
+        dst[static_cast<int64_t>(e) * a.page_size] = static_cast<uint16_t>(vrows[i][e >> 1] >> 16 * (e & 1));
+    }
+  }
+  if (!is_v || !run) return;
+  uint16_t* dst = base + ((static_cast<int64_t>(page_s[0]) * heads + head) * dim + e0) * a.page_size + off_s[0];
+#pragma unroll
+  for (int e = 0; e < 8; ++e) {
+    conv_u32x4 lo, hi;  // channel e of rows 0 .. 7 and 8 .. 15
+#pragma unroll
+    for (int p = 0; p < 4; ++p) {
+      const int sh = 16 * (e & 1);
+      lo[p] = (vrows[2 * p][e >> 1] >> sh & 0xffffu) | (vrows[2 * p + 1][e >> 1] >> sh) << 16;
+      hi[p] = (vrows[2 * p + 8][e >> 1] >> sh & 0xffffu) | (vrows[2 * p + 9][e >> 1] >> sh) << 16;
+    }
+    *reinterpret_cast<conv_u32x4*>(dst + static_cast<int64_t>(e) * a.page_size) = lo;
+    *reinterpret_cast<conv_u32x4*>(dst + static_cast<int64_t>(e) * a.page_size + 8) = hi;
+  }
+}
+
 // q_channels, k_channels: multiples of head_dim; v_channels: a multiple of value_dim.  `slots` null: k and v go to
 // plain rows.  `dtype`: the type of in, out_q, out_k, out_v (and of the cache).  `wt` float32 [taps, channels] and
-// `bias_f` float32 [channels]: copies of `w` and `bias` for the 16-byte form, or null.
+// `bias_f` float32 [channels]: copies of `w` and `bias` for the 16-byte form, or null.  `requests`: the step's (q_start
+// holds one entry more).
 extern "C" int ix_short_conv(const void* in, int dtype, int64_t in_stride, const void* bias, int bias_dtype,
                              const void* w, int w_dtype, int taps, float* state, int64_t state_stride,
                              const int32_t* seq_of_token, const int32_t* q_start, const int32_t* state_slots,
                              const float* cos_sin, int rot_dims, int silu, const int32_t* slots, int page_size,
                              void* out_q, void* out_k, void* out_v, int64_t tokens, int q_channels, int k_channels,
                              int v_channels, int head_dim, int value_dim, const float* wt, const float* bias_f,
-                             const int32_t* positions, float temp_coef, float temp_every, hipStream_t stream) {
+                             const int32_t* positions, float temp_coef, float temp_every, int requests,
+                             hipStream_t stream) {
   IX_REQUIRE(tokens >= 0 && taps >= 1 && taps <= 64, "between 1 and 64 taps");
   IX_REQUIRE(head_dim > 0 && value_dim > 0 && q_channels >= 0 && k_channels >= 0 && v_channels >= 0,
              "sizes must be positive");
@@ -419,6 +571,18 @@ extern "C" int ix_short_conv(const void* in, int dtype, int64_t in_stride, const
       value_dim % 8 == 0 && rot_dims % 16 == 0 && in_stride % 8 == 0 && state_stride % 4 == 0 && aligned(in) &&
       aligned(state) && aligned(wt) && aligned(bias_f) && aligned(out_q) && aligned(out_k) && plain_rows_ok &&
       (slots == nullptr || aligned(out_k))) {
+    if (rot_dims == 0 && taps <= 4 && tokens >= 64 && tokens >= 8 * static_cast<int64_t>(requests) && aligned(out_v)) {
+      const int units = channels / 8, tiles = static_cast<int>((tokens + CONV_TILE - 1) / CONV_TILE);
+      dim3 tgrid(tiles + requests, (units + CONV_TILE_THREADS - 1) / CONV_TILE_THREADS);
+#define CASE(TAPS)                                                                                                \
+  case TAPS:                                                                                                      \
+    hipLaunchKernelGGL(short_conv_tile_kernel<TAPS>, tgrid, dim3(CONV_TILE_THREADS), 0, stream, a, wt,            \
+                       bias ? bias_f : nullptr, units, requests, static_cast<int>(tokens));                         \
+    break;
+      switch (taps) { CASE(1) CASE(2) CASE(3) CASE(4) }
+#undef CASE
+      return ix_check_launch("ix_short_conv");
+    }
     const int vunits = (q_channels + k_channels) / head_dim * (head_dim / 8 - rot_dims / 16) + v_channels / 8;
     dim3 vgrid(static_cast<unsigned>(tokens), (vunits + CONV_THREADS - 1) / CONV_THREADS);
     hipLaunchKernelGGL(short_conv_vec8_kernel, vgrid, block, 0, stream, a, wt, bias ? bias_f : nullptr, vunits);

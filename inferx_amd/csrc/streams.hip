@@ -205,6 +205,40 @@ embed_norm_kernel(float* __restrict__ h, const TW* __restrict__ table, const int
   }
 }
 
+// the same with the row in registers, four columns per thread and turn
+template <typename TW, int PER>
+__global__ void __launch_bounds__(1024)
+embed_norm_vec4_kernel(float* __restrict__ h, const TW* __restrict__ table, const int32_t* __restrict__ ids,
+                       const float* __restrict__ weight, int width, int64_t vocab, int streams, float scale, float eps) {
+  __shared__ float red[16];
+  const int64_t t = blockIdx.x;
+  const int64_t id = ids[t];
+  const bool ok = id >= 0 && id < vocab;
+  const TW* row = table + (ok ? id : 0) * width;
+  float4 x[PER];
+  float ss = 0.f;
+#pragma unroll
+  for (int p = 0; p < PER; ++p) {
+    const int c = 4 * (p * blockDim.x + threadIdx.x);
+    x[p] = c < width ? st_load4(row + c) : float4{0.f, 0.f, 0.f, 0.f};
+    x[p] = float4{x[p].x * scale, x[p].y * scale, x[p].z * scale, x[p].w * scale};
+    ss += x[p].x * x[p].x + x[p].y * x[p].y + x[p].z * x[p].z + x[p].w * x[p].w;
+  }
+  float inv = ok ? 1.0f : 0.f;
+  if (weight) {
+    ss = ix_block_sum(ss, red);
+    inv = ok ? 1.0f / sqrtf(ss / static_cast<float>(width) + eps) : 0.f;
+  }
+#pragma unroll
+  for (int p = 0; p < PER; ++p) {
+    const int c = 4 * (p * blockDim.x + threadIdx.x);
+    if (c >= width) continue;
+    const float4 w = weight ? st_load4(weight + c) : float4{1.f, 1.f, 1.f, 1.f};
+    const float4 v = float4{x[p].x * inv * w.x, x[p].y * inv * w.y, x[p].z * inv * w.z, x[p].w * inv * w.w};
+    for (int j = 0; j < streams; ++j) st_store4(h + (t * streams + j) * width + c, v);
+  }
+}
+
 extern "C" int ix_embed_norm(float* h, const void* table, int table_dtype, const int32_t* ids, const float* weight,
                              int64_t tokens, int64_t width, int64_t vocab, int streams, float scale, float eps,
                              hipStream_t stream) {
@@ -213,6 +247,24 @@ extern "C" int ix_embed_norm(float* h, const void* table, int table_dtype, const
   IX_REQUIRE(tokens < (1ll << 31), "too many tokens for one launch");
   if (tokens == 0) return 0;
   dim3 grid(static_cast<unsigned>(tokens)), block(256);
+  const uintptr_t all = reinterpret_cast<uintptr_t>(h) | reinterpret_cast<uintptr_t>(table) | reinterpret_cast<uintptr_t>(weight);
+  if (width % 4 == 0 && width <= 16384 && (all & 15) == 0) {
+    const int quads = static_cast<int>(width / 4);
+    int threads = 64;
+    while (threads < 1024 && threads < quads) threads *= 2;
+    const int per = (quads + threads - 1) / threads;
+#define LAUNCH(T, PER)                                                                                                  \
+  hipLaunchKernelGGL((embed_norm_vec4_kernel<T, PER>), grid, dim3(threads), 0, stream, h, (const T*)table, ids, weight, \
+                     static_cast<int>(width), vocab, streams, scale, eps)
+#define BY_PER(T)                  \
+  if (per == 1) LAUNCH(T, 1);      \
+  else if (per == 2) LAUNCH(T, 2); \
+  else LAUNCH(T, 4)
+    if (table_dtype == IX_F32) { BY_PER(float); } else { BY_PER(bf16_t); }
+#undef BY_PER
+#undef LAUNCH
+    return ix_check_launch("ix_embed_norm");
+  }
   if (table_dtype == IX_F32)
     hipLaunchKernelGGL(embed_norm_kernel<float>, grid, block, 0, stream, h, (const float*)table, ids, weight, width, vocab,
                        streams, scale, eps);

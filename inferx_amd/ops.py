@@ -1136,7 +1136,7 @@ def short_conv(x: torch.Tensor, bias: Optional[torch.Tensor], weight: torch.Tens
           _i64(state.stride(0)), _ptr(rows.seq_of_token), _ptr(rows.q_start), _ptr(rows.state_slots), _ptr(cos_sin),
           _i32(rot), _i32(1 if silu else 0), _ptr(slots), _i32(page_size), _ptr(out_q), _ptr(out_k), _ptr(out_v),
           _i64(T), _i32(cq), _i32(ck), _i32(cv), _i32(d), _i32(vd), _ptr(weight_t), _ptr(bias_f32), _ptr(positions), _f32(coef),
-          _f32(every), _stream())
+          _f32(every), _i32(rows.q_start.numel() - 1), _stream())
 
 
 def delta_rule(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, ab: torch.Tensor, a_log: torch.Tensor,

@@ -66,7 +66,7 @@ def test_embedding_with_a_norm_starts_every_copy(streams, width, dtype):
                                                      (2, 1, 32, 32, 1, (0.3, 5), True), (8, 2, 64, 64, 4, None, True),
                                                      (4, 2, 16, 16, 3, (0.5, 7), False), (2, 2, 7, 7, 5, (0.2, 3), False)])
 def test_convolution_with_a_query_temperature(H, G, d, vd, taps, temp, keys, dtype, tol):
-    """Requests in portions of changing size (a whole prompt, two tokens, one), slots out of order, the state carried;
+    """Requests in portions of changing size (down to two tokens and one, up to several tiles of rows), slots out of order, the state carried;
     the first token whose count reaches a multiple of the step, and the one before; queries alone (no keys of its own)."""
     from inferx_amd.parts.short_conv import ShortConv
     names = ("q", "k", "v") if keys else ("q",)
@@ -76,16 +76,16 @@ def test_convolution_with_a_query_temperature(H, G, d, vd, taps, temp, keys, dty
     conv = ShortConv(cq, ck, cv, d, vd, taps)
     at = {"q": slice(0, cq), "k": slice(cq, cq + ck), "v": slice(cq + ck, C)}
     conv.bind({f"{n}.conv": w[at[n]].to(DEV) for n in names}, names=names, bias=bias.to(DEV))
-    lengths = [30, 23, 18]
+    lengths = [110, 40, 60]
     x = [rnd((n, C + 8), 10 + i, 1.0, dtype) for i, n in enumerate(lengths)]  # rows longer than the channels: a gate behind
     state = torch.full((4, max(1, (taps - 1) * C)), float("nan"), device=DEV)
     slots = [2, 0, 3]
     state[slots] = 0
     page = 16
-    kc, vc = torch.zeros(8, G, page, d, dtype=dtype, device=DEV), torch.zeros(8, G, vd, page, dtype=dtype, device=DEV)
-    first_slot = [0, 32, 64]
+    kc, vc = torch.zeros(16, G, page, d, dtype=dtype, device=DEV), torch.zeros(16, G, vd, page, dtype=dtype, device=DEV)
+    first_slot = [0, 112, 160]
     done, got = [0, 0, 0], [[], [], []]
-    for portions in ((7, 23, 1), (1, 0, 1), (2, 0, 2), (20, 0, 14)):
+    for portions in ((7, 31, 1), (1, 0, 1), (8, 0, 2), (94, 9, 56)):
         rows = step_rows(portions, slots)
         pos = np.concatenate([np.arange(a, a + n) for a, n in zip(done, portions)]).astype(np.int32)
         cache_slots = np.concatenate([f + np.arange(a, a + n) for f, a, n in zip(first_slot, done, portions)]).astype(np.int32)
