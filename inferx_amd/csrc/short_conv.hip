@@ -378,12 +378,12 @@ __global__ void __launch_bounds__(CONV_THREADS) short_conv_vec8_kernel(ConvArgs 
   }
 }
 
-// The same for prompt portions without a rotation, at most four taps: a thread owns eight channels of sixteen
-// consecutive rows, so that taps, bias and every input are read once, and values that sixteen consecutive places of a
-// page take are written sixteen at a time.  A row whose inputs all lie in its own portion (its place i >= taps - 1) is
+// The same for prompt portions without a rotation, at most four taps: a thread owns eight channels of eight
+// consecutive rows, so that taps, bias and nearly every input are read once, and values that eight consecutive places of
+// a page take are written eight at a time.  A row whose inputs all lie in its own portion (its place i >= taps - 1) is
 // formed here; the portion's first rows, a last row that is among them, and the new state belong to one further
 // workgroup per request (blockIdx.x < requests), which alone reads and writes the state.
-#define CONV_TILE 16
+#define CONV_TILE 8
 #define CONV_TILE_THREADS 128
 
 template <int TAPS>
@@ -439,7 +439,7 @@ short_conv_tile_kernel(ConvArgs a, const float* __restrict__ wt, const float* __
     return;
   }
   const int r0 = (static_cast<int>(blockIdx.x) - requests) * CONV_TILE;
-  conv_u32x4 raw[CONV_TILE + TAPS - 1];  // the inputs of rows r0 - (taps - 1) .. r0 + 15
+  conv_u32x4 raw[CONV_TILE + TAPS - 1];  // the inputs of rows r0 - (taps - 1) .. r0 + CONV_TILE - 1
 #pragma unroll
   for (int i = 0; i < CONV_TILE + TAPS - 1; ++i)
     raw[i] = *reinterpret_cast<const conv_u32x4*>(in + static_cast<int64_t>(min(max(r0 - (TAPS - 1) + i, 0), tokens - 1)) * a.in_stride + c0);
@@ -451,7 +451,7 @@ short_conv_tile_kernel(ConvArgs a, const float* __restrict__ wt, const float* __
 #pragma unroll
   for (int e = 0; e < 8; ++e) b[e] = bias_f ? bias_f[c0 + e] : 0.f;
   // what the workgroup needs to know of its rows, a row per lane: whether it is formed here, its place in the cache, its
-  // temperature; and whether all sixteen places lie side by side on one page
+  // temperature; and whether all the places lie side by side on one page
   if (threadIdx.x < CONV_TILE) {
     const int i = threadIdx.x, row = min(r0 + i, tokens - 1);
     const bool formed = r0 + i < tokens && row - a.q_start[a.seq_of_token[row]] >= TAPS - 1;
@@ -464,7 +464,7 @@ short_conv_tile_kernel(ConvArgs a, const float* __restrict__ wt, const float* __
     const bool beside = a.slots && a.page_size % 8 == 0 && slot0 % 8 == 0 && formed && slot == slot0 + i &&
                         off + CONV_TILE - i <= a.page_size && off >= i;
     const uint64_t all = __ballot(beside);
-    if (i == 0) run_s = (all & 0xffffu) == 0xffffu;
+    if (i == 0) run_s = all == (1ull << CONV_TILE) - 1;
   }
   __syncthreads();
   if (!live) return;
@@ -516,15 +516,16 @@ short_conv_tile_kernel(ConvArgs a, const float* __restrict__ wt, const float* __
   uint16_t* dst = base + ((static_cast<int64_t>(page_s[0]) * heads + head) * dim + e0) * a.page_size + off_s[0];
 #pragma unroll
   for (int e = 0; e < 8; ++e) {
-    conv_u32x4 lo, hi;  // channel e of rows 0 .. 7 and 8 .. 15
 #pragma unroll
-    for (int p = 0; p < 4; ++p) {
-      const int sh = 16 * (e & 1);
-      lo[p] = (vrows[2 * p][e >> 1] >> sh & 0xffffu) | (vrows[2 * p + 1][e >> 1] >> sh) << 16;
-      hi[p] = (vrows[2 * p + 8][e >> 1] >> sh & 0xffffu) | (vrows[2 * p + 9][e >> 1] >> sh) << 16;
+    for (int r = 0; r < CONV_TILE; r += 8) {
+      conv_u32x4 x;  // channel e of rows r .. r + 7
+#pragma unroll
+      for (int p = 0; p < 4; ++p) {
+        const int sh = 16 * (e & 1);
+        x[p] = (vrows[r + 2 * p][e >> 1] >> sh & 0xffffu) | (vrows[r + 2 * p + 1][e >> 1] >> sh) << 16;
+      }
+      *reinterpret_cast<conv_u32x4*>(dst + static_cast<int64_t>(e) * a.page_size + r) = x;
     }
-    *reinterpret_cast<conv_u32x4*>(dst + static_cast<int64_t>(e) * a.page_size) = lo;
-    *reinterpret_cast<conv_u32x4*>(dst + static_cast<int64_t>(e) * a.page_size + 8) = hi;
   }
 }
 
