@@ -37,7 +37,8 @@ typedef float f32x4 __attribute__((ext_vector_type(4)));
 
 // head_dim = 16 * NB; a tile holds up to 16 * QT queries; PF: request the next iteration's keys and values
 // before this iteration's are multiplied (pays when few wavefronts are resident: decoding)
-template <int NB, int QT, bool PF, bool GQ = false>
+// MORE false: without capped scores and a gate (for the plain decoding steps, where a test a round is measurable)
+template <int NB, int QT, bool PF, bool GQ = false, bool MORE = true>
 __global__ void __launch_bounds__(256)
 attn_mfma_kernel(const __bf16* __restrict__ q, const __bf16* __restrict__ k_cache, const __bf16* __restrict__ v_cache,
                  const int32_t* __restrict__ block_table, const int32_t* __restrict__ tile_seq,
@@ -205,8 +206,9 @@ attn_mfma_kernel(const __bf16* __restrict__ q, const __bf16* __restrict__ k_cach
       // scores stay unscaled: the scale (times log2 e) enters with the reference point in one fused multiply-add
       float sv[8];
       float mx = -INFINITY;
-      const float sl = cap2 > 0.f ? 1.0f : scale_log2;
-      if (cap2 > 0.f) {  // (uniform; capped scores are in units of log2 already)
+      const bool capped = MORE && cap2 > 0.f;
+      const float sl = capped ? 1.0f : scale_log2;
+      if (capped) {  // (uniform; capped scores are in units of log2 already)
 #pragma unroll
         for (int b = 0; b < 2; ++b)
 #pragma unroll
@@ -291,7 +293,7 @@ attn_mfma_kernel(const __bf16* __restrict__ q, const __bf16* __restrict__ k_cach
       for (int b = 0; b < NB; ++b) {
         bf16x4 v;
         f32x4 by = f32x4{inv, inv, inv, inv};
-        if (gate) {
+        if (MORE && gate) {
           const bf16x4 gv = *reinterpret_cast<const bf16x4*>(gate + token * gate_stride + head * D + 4 * g + 16 * b);
 #pragma unroll
           for (int i = 0; i < 4; ++i) by[i] = inv * __builtin_amdgcn_rcpf(1.0f + __expf(-(float)gv[i]));
@@ -374,7 +376,7 @@ int ix_attention_combine(const float* part_o, const float* part_ml, void* out, i
   return ix_check_launch("ix_attention_combine");
 }
 
-template <int NB, int QT, bool PF, bool GQ = false>
+template <int NB, int QT, bool PF, bool GQ = false, bool MORE = true>
 static void launch_attn(dim3 grid, hipStream_t stream, const void* q, const void* k, const void* v,
                         const int32_t* table, const int32_t* tile_seq, const int32_t* tile_q0,
                         const int32_t* tile_rows, const int32_t* positions, void* out, float* part_o, float* part_ml,
@@ -389,7 +391,7 @@ static void launch_attn(dim3 grid, hipStream_t stream, const void* q, const void
   const int64_t waves = static_cast<int64_t>(n_tiles) * n_splits * grid.y;
   const int per_group = waves >= 4 * 512 ? 4 : (waves >= 2 * 512 ? 2 : 1);
   grid.x = static_cast<unsigned>((static_cast<int64_t>(n_tiles) * n_splits + per_group - 1) / per_group);
-  hipLaunchKernelGGL((attn_mfma_kernel<NB, QT, PF, GQ>), grid, dim3(64 * per_group), 0, stream, (const __bf16*)q, (const __bf16*)k,
+  hipLaunchKernelGGL((attn_mfma_kernel<NB, QT, PF, GQ, MORE>), grid, dim3(64 * per_group), 0, stream, (const __bf16*)q, (const __bf16*)k,
                      (const __bf16*)v, table, tile_seq, tile_q0, tile_rows, positions, (__bf16*)out, part_o, part_ml,
                      n_tiles, n_splits, heads, kv_heads, page_size, max_blocks, scale_log2, window, page_shift, sink,
                      reinterpret_cast<const float2*>(turn_back), cap_slope, cap2, (const __bf16*)gate, gate_stride);
@@ -426,6 +428,7 @@ static int attention_mfma_any(const void* q, const void* k_cache, const void* v_
   dim3 grid(static_cast<unsigned>((units + 3) / 4), grouped ? kv_heads : heads);
   const float scale_log2 = scale * 1.4426950408889634f;
   const float cap2 = softcap * 1.4426950408889634f, cap_slope = softcap > 0.f ? 2.0f * scale_log2 / softcap : 0.f;
+  const bool more = softcap > 0.f || gate != nullptr;
 #define ARGS                                                                                                    \
   grid, stream, q, k_cache, v_cache, block_table, tile_seq, tile_q0, tile_rows, positions, out, part_o, part_ml, \
       n_tiles, n_splits, heads, kv_heads, page_size, max_blocks, scale_log2, window, sink, turn_back, cap_slope,    \
@@ -433,9 +436,11 @@ static int attention_mfma_any(const void* q, const void* k_cache, const void* v_
 #define CASE(NB)                                                    \
   case NB:                                                          \
     if (grouped) {                                                  \
-      if (prefetch) launch_attn<NB, 1, true, true>(ARGS);           \
+      if (prefetch && more) launch_attn<NB, 1, true, true>(ARGS);   \
+      else if (prefetch) launch_attn<NB, 1, true, true, false>(ARGS); \
       else launch_attn<NB, 1, false, true>(ARGS);                   \
-    } else if (prefetch) launch_attn<NB, 1, true>(ARGS);            \
+    } else if (prefetch && more) launch_attn<NB, 1, true>(ARGS);    \
+    else if (prefetch) launch_attn<NB, 1, true, false, false>(ARGS); \
     else launch_attn<NB, 1, false>(ARGS);                           \
     break;
 #define CASE4(NB)                        \
