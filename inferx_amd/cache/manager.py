@@ -14,7 +14,9 @@ A page group is a set of cache-owning layer executions with the same need (kv
 heads, head size, window).  Every group has pages of its own: its own pool, its
 own block list per request.  A group with window W gives a page back as soon as
 no query at or after the request's next position can read it: page j (tokens
-[j*P, (j+1)*P)) is dead once (j+1)*P <= cached + 1 - W.  The reference keeps
+[j*P, (j+1)*P)) is dead once (j+1)*P <= cached + 1 - W.  A group in chunks of C
+positions (a query reads its own chunk only) gives a page back as soon as the next
+position's chunk starts after it: (j+1)*P <= cached - cached % C.  The reference keeps
 every token of its windowed layers (src/model/gpt_oss.cc:259-262); releasing
 is this engine's own rule.
 
@@ -142,16 +144,18 @@ class GroupLayout:
     pages that the window has passed until the request ends (what the reference does for its windowed layers,
     src/model/gpt_oss.cc:259-262); the attention kernels mask by the window either way, so the two settings must
     give the same logits, which is what the switch is for.  `keep_first`: the pages that hold a request's first
-    `keep_first` tokens are never given back (a window whose queries also read those tokens)."""
+    `keep_first` tokens are never given back (a window whose queries also read those tokens).  `chunk` C > 0 (then without
+    a window): only the tokens of the chunk of C positions that the next position lies in are kept."""
 
     window: int = 0
     release_passed: bool = True
     keep_first: int = 0
+    chunk: int = 0
 
     @property
     def release_window(self) -> int:
-        """The window as the bookkeeping sees it: 0 if no page is ever given back early."""
-        return self.window if self.release_passed else 0
+        """The window as the bookkeeping sees it: 0 if no page is ever given back early, negative for chunks."""
+        return (self.window or -self.chunk) if self.release_passed else 0
 
 
 class _PoolView:
@@ -188,7 +192,8 @@ def pages_for_window(window: int, page_size: int, max_requests: int, max_step_to
     """Pages that a windowed group can ever hold at once when no step brings more than `max_step_tokens` tokens
     of a request: per request the pages that cover the window behind its next position and the step in front of
     it (plus the two that the ends may straddle) and the pages of the `keep_first` tokens that are never given
-    back, for every request slot.  A pool of this size never runs out."""
+    back, for every request slot.  A pool of this size never runs out.  (A chunk keeps no more than a window of its
+    size.)"""
     return max_requests * (-(-(window + max_step_tokens) // page_size) + 2 + -(-keep_first // page_size))
 
 

@@ -14,9 +14,11 @@ from . import gosuvik  # registers Gosuvik
 from .gosuvik import GosuvikConfig
 from . import setopel  # registers Setopel
 from .setopel import SetopelConfig
+from . import zevivik  # registers Zevivik
+from .zevivik import ZevivikConfig
 
 __all__ = [
     "ConfigError", "config_class_for", "config_from_dict", "config_from_directory", "config_from_json",
     "known_architectures", "register_architecture", "LayerSpec", "ModelSpec", "PartSpec", "ScheduleEntry", "linear_head", "token_embedding",
-    "Qwen2MoeConfig", "PelalixConfig", "DezudraConfig", "BibevikConfig", "GosuvikConfig", "SetopelConfig",
+    "Qwen2MoeConfig", "PelalixConfig", "DezudraConfig", "BibevikConfig", "GosuvikConfig", "SetopelConfig", "ZevivikConfig",
 ]

@@ -51,10 +51,13 @@ class ScheduleEntry:
     """One execution of a layer.  `layer` indexes `ModelSpec.layers` (a layer
     may be named by several entries: shared weights, separate caches).
     `cache_from` names an EARLIER entry whose cache this execution reads
-    instead of owning one (it then writes nothing)."""
+    instead of owning one (it then writes nothing).  `enter` (kind "entry"): a
+    part that the residual stream passes right before this execution (what a
+    loop adds at the start of each pass)."""
 
     layer: int
     cache_from: Optional[int] = None
+    enter: Optional[PartSpec] = None
 
 
 @dataclass(frozen=True)

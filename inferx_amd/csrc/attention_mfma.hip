@@ -1,7 +1,8 @@
 // Paged attention on the matrix cores (bfloat16), for prompt portions and for
 // decoding alike.  Same arithmetic as the plain kernel (attention_plain.hip):
 // keys [start, p] through the block table, scores * scale, softmax online in
-// float32, PV accumulated in float32.
+// float32, PV accumulated in float32; `start` by `span` (0, a window or chunks:
+// ix_first_key in common.h).
 //
 // Unit of work = one wavefront: a tile of up to 16 consecutive queries of one
 // request and one query head, over one slice of that tile's keys (split-KV).
@@ -45,7 +46,7 @@ attn_mfma_kernel(const __bf16* __restrict__ q, const __bf16* __restrict__ k_cach
                  const int32_t* __restrict__ tile_q0, const int32_t* __restrict__ tile_rows,
                  const int32_t* __restrict__ positions, __bf16* __restrict__ out, float* __restrict__ part_o,
                  float* __restrict__ part_ml, int n_tiles, int n_splits, int heads, int kv_heads, int page_size,
-                 int max_blocks, float scale_log2, int window, int page_shift, const float* __restrict__ sink,
+                 int max_blocks, float scale_log2, int span, int page_shift, const float* __restrict__ sink,
                  const float2* __restrict__ turn_back, float cap_slope, float cap2, const __bf16* __restrict__ gate,
                  int64_t gate_stride) {
   // sink (one float per head, or null): exp(sink) joins the softmax's denominator, with no key and no value, not
@@ -73,7 +74,7 @@ attn_mfma_kernel(const __bf16* __restrict__ q, const __bf16* __restrict__ k_cach
   const int32_t* table = block_table + static_cast<int64_t>(tile_seq[tile]) * max_blocks;
 
   // keys this tile reads at all: [lo, hi); this wavefront's slice [ks, ke)
-  const int lo = (window > 0 && pos0 + 1 > window) ? pos0 + 1 - window : 0;
+  const int lo = ix_first_key(pos0, span);
   const int hi = pos0 + (GQ ? 1 : rows);
   const int lo_al = lo & ~(ATTN_KEYS_PER_ITER - 1);
   const int per = (((hi - lo_al + n_splits - 1) / n_splits) + ATTN_KEYS_PER_ITER - 1) & ~(ATTN_KEYS_PER_ITER - 1);
@@ -96,6 +97,12 @@ attn_mfma_kernel(const __bf16* __restrict__ q, const __bf16* __restrict__ k_cach
 
   f32x4 o[QT][NB];
   float m[QT], lsum[QT];
+  int first[QT], last_first[QT];  // the first key that this lane's query reads, and the last query of the sixteen
+#pragma unroll
+  for (int t = 0; t < QT; ++t) {
+    first[t] = GQ ? lo : ix_first_key(pos0 + 16 * t + n, span);
+    last_first[t] = GQ ? lo : ix_first_key(pos0 + 16 * t + 15, span);
+  }
 #pragma unroll
   for (int t = 0; t < QT; ++t) {
     const bool sunk = sink != nullptr && split == 0;
@@ -202,7 +209,7 @@ attn_mfma_kernel(const __bf16* __restrict__ q, const __bf16* __restrict__ k_cach
       // ---- mask, online softmax for this lane's query over its 8 keys ----
       const int my_pos = pos0 + (GQ ? 0 : 16 * t + n);
       const bool my_row = 16 * t + n < rows;
-      const int my_lo = (window > 0 && my_pos + 1 > window) ? my_pos + 1 - window : 0;
+      const int my_lo = first[t];
       // scores stay unscaled: the scale (times log2 e) enters with the reference point in one fused multiply-add
       float sv[8];
       float mx = -INFINITY;
@@ -218,7 +225,7 @@ attn_mfma_kernel(const __bf16* __restrict__ q, const __bf16* __restrict__ k_cach
       // (GQ: the columns without a query head hold zeros for q; what they sum is not stored)
       const bool inner = (GQ || 16 * t + 16 <= rows) && kb + ATTN_KEYS_PER_ITER <= ke &&
                          kb + ATTN_KEYS_PER_ITER - 1 <= pos0 + (GQ ? 0 : 16 * t) &&
-                         (window == 0 || kb > pos0 + (GQ ? 0 : 16 * t + 15) - window);
+                         kb >= last_first[t];
       if (inner) {
 #pragma unroll
         for (int j = 0; j < 8; ++j) {
@@ -321,7 +328,8 @@ attn_mfma_kernel(const __bf16* __restrict__ q, const __bf16* __restrict__ k_cach
 __global__ void __launch_bounds__(128)
 attn_combine_kernel(const float* __restrict__ part_o, const float* __restrict__ part_ml, __bf16* __restrict__ out,
                     int n_splits, int head_dim, int heads, const float2* __restrict__ turn_back,
-                    const __bf16* __restrict__ gate, int64_t gate_stride) {
+                    const __bf16* __restrict__ gate, int64_t gate_stride, const __bf16* __restrict__ head_gate,
+                    int64_t head_gate_stride) {
   __shared__ float wgt[256];
   __shared__ float inv_l;
   const int64_t th = blockIdx.x;  // token * heads + head
@@ -338,7 +346,8 @@ attn_combine_kernel(const float* __restrict__ part_o, const float* __restrict__ 
       lloc += w * ml[2 * s + 1];
     }
     const float L = ix_wave_sum(lloc);
-    if (threadIdx.x == 0) inv_l = 1.0f / L;
+    if (threadIdx.x == 0)
+      inv_l = head_gate ? 1.0f / (L * (1.0f + __expf(-(float)head_gate[(th / heads) * head_gate_stride + th % heads]))) : 1.0f / L;
   }
   __syncthreads();
   const float* po = part_o + th * n_splits * head_dim;
@@ -369,10 +378,10 @@ attn_combine_kernel(const float* __restrict__ part_o, const float* __restrict__ 
 
 int ix_attention_combine(const float* part_o, const float* part_ml, void* out, int64_t tokens, int heads,
                          int n_splits, int head_dim, hipStream_t stream, const float* turn_back, const void* gate,
-                         int64_t gate_stride) {
+                         int64_t gate_stride, const void* head_gate, int64_t head_gate_stride) {
   hipLaunchKernelGGL(attn_combine_kernel, dim3(static_cast<unsigned>(tokens * heads)), dim3(128), 0, stream, part_o,
                      part_ml, (__bf16*)out, n_splits, head_dim, heads, reinterpret_cast<const float2*>(turn_back),
-                     (const __bf16*)gate, gate_stride);
+                     (const __bf16*)gate, gate_stride, (const __bf16*)head_gate, head_gate_stride);
   return ix_check_launch("ix_attention_combine");
 }
 
@@ -381,7 +390,7 @@ static void launch_attn(dim3 grid, hipStream_t stream, const void* q, const void
                         const int32_t* table, const int32_t* tile_seq, const int32_t* tile_q0,
                         const int32_t* tile_rows, const int32_t* positions, void* out, float* part_o, float* part_ml,
                         int n_tiles, int n_splits, int heads, int kv_heads, int page_size, int max_blocks,
-                        float scale_log2, int window, const float* sink, const float* turn_back, float cap_slope,
+                        float scale_log2, int span, const float* sink, const float* turn_back, float cap_slope,
                         float cap2, const void* gate, int64_t gate_stride) {
   int page_shift = -1;  // log2 of the page size if it is a power of two
   for (int b = 4; b < 31; ++b)
@@ -393,7 +402,7 @@ static void launch_attn(dim3 grid, hipStream_t stream, const void* q, const void
   grid.x = static_cast<unsigned>((static_cast<int64_t>(n_tiles) * n_splits + per_group - 1) / per_group);
   hipLaunchKernelGGL((attn_mfma_kernel<NB, QT, PF, GQ, MORE>), grid, dim3(64 * per_group), 0, stream, (const __bf16*)q, (const __bf16*)k,
                      (const __bf16*)v, table, tile_seq, tile_q0, tile_rows, positions, (__bf16*)out, part_o, part_ml,
-                     n_tiles, n_splits, heads, kv_heads, page_size, max_blocks, scale_log2, window, page_shift, sink,
+                     n_tiles, n_splits, heads, kv_heads, page_size, max_blocks, scale_log2, span, page_shift, sink,
                      reinterpret_cast<const float2*>(turn_back), cap_slope, cap2, (const __bf16*)gate, gate_stride);
 }
 
@@ -405,7 +414,7 @@ static int attention_mfma_any(const void* q, const void* k_cache, const void* v_
                               const int32_t* tile_seq, const int32_t* tile_q0, const int32_t* tile_rows,
                               const int32_t* positions, void* out, float* part_o, float* part_ml, int64_t tokens,
                               int n_tiles, int tile_queries, int n_splits, int heads, int kv_heads, int head_dim,
-                              int page_size, int max_blocks, float scale, int window, int prefetch, int grouped,
+                              int page_size, int max_blocks, float scale, int span, int prefetch, int grouped,
                               const float* sink, const float* turn_back, float softcap, const void* gate,
                               int64_t gate_stride, hipStream_t stream) {
   IX_REQUIRE(softcap >= 0.f, "the cap of the scores must not be negative");
@@ -419,7 +428,6 @@ static int attention_mfma_any(const void* q, const void* k_cache, const void* v_
   IX_REQUIRE(page_size % 16 == 0 && page_size > 0, "page_size must be a multiple of 16");
   IX_REQUIRE(n_splits >= 1 && n_splits <= 256, "n_splits must be between 1 and 256");
   IX_REQUIRE(n_splits == 1 || (part_o != nullptr && part_ml != nullptr), "workspace needed for split keys");
-  IX_REQUIRE(window >= 0, "window must not be negative");
   IX_REQUIRE(heads <= 65535, "too many heads");
   IX_REQUIRE(!grouped || (tile_queries == 16 && heads / kv_heads <= 16),
              "grouped queries: tiles of 16, at most 16 query heads per key/value head");
@@ -431,7 +439,7 @@ static int attention_mfma_any(const void* q, const void* k_cache, const void* v_
   const bool more = softcap > 0.f || gate != nullptr;
 #define ARGS                                                                                                    \
   grid, stream, q, k_cache, v_cache, block_table, tile_seq, tile_q0, tile_rows, positions, out, part_o, part_ml, \
-      n_tiles, n_splits, heads, kv_heads, page_size, max_blocks, scale_log2, window, sink, turn_back, cap_slope,    \
+      n_tiles, n_splits, heads, kv_heads, page_size, max_blocks, scale_log2, span, sink, turn_back, cap_slope,    \
       cap2, gate, gate_stride
 #define CASE(NB)                                                    \
   case NB:                                                          \
@@ -471,11 +479,11 @@ extern "C" int ix_attention_mfma(const void* q, const void* k_cache, const void*
                                  const int32_t* tile_seq, const int32_t* tile_q0, const int32_t* tile_rows,
                                  const int32_t* positions, void* out, float* part_o, float* part_ml, int64_t tokens,
                                  int n_tiles, int tile_queries, int n_splits, int heads, int kv_heads, int head_dim,
-                                 int page_size, int max_blocks, float scale, int window, int prefetch, int grouped,
+                                 int page_size, int max_blocks, float scale, int span, int prefetch, int grouped,
                                  hipStream_t stream) {
   return attention_mfma_any(q, k_cache, v_cache, block_table, tile_seq, tile_q0, tile_rows, positions, out, part_o,
                             part_ml, tokens, n_tiles, tile_queries, n_splits, heads, kv_heads, head_dim, page_size,
-                            max_blocks, scale, window, prefetch, grouped, nullptr, nullptr, 0.f, nullptr, 0, stream);
+                            max_blocks, scale, span, prefetch, grouped, nullptr, nullptr, 0.f, nullptr, 0, stream);
 }
 
 // The same with a sink per head (float32 [heads], or null) in every softmax's denominator, and with the result of
@@ -487,11 +495,11 @@ extern "C" int ix_attention_mfma_sink(const void* q, const void* k_cache, const 
                                       const int32_t* tile_rows, const int32_t* positions, void* out, float* part_o,
                                       float* part_ml, int64_t tokens, int n_tiles, int tile_queries, int n_splits,
                                       int heads, int kv_heads, int head_dim, int page_size, int max_blocks, float scale,
-                                      int window, int prefetch, int grouped, const float* sink, const float* turn_back,
+                                      int span, int prefetch, int grouped, const float* sink, const float* turn_back,
                                       float softcap, const void* gate, int64_t gate_stride, hipStream_t stream) {
   return attention_mfma_any(q, k_cache, v_cache, block_table, tile_seq, tile_q0, tile_rows, positions, out, part_o,
                             part_ml, tokens, n_tiles, tile_queries, n_splits, heads, kv_heads, head_dim, page_size,
-                            max_blocks, scale, window, prefetch, grouped, sink, turn_back, softcap, gate, gate_stride, stream);
+                            max_blocks, scale, span, prefetch, grouped, sink, turn_back, softcap, gate, gate_stride, stream);
 }
 
 // ---- the same operation without a workspace argument -----------------------------------------------------------
@@ -535,7 +543,7 @@ extern "C" int ix_attention_mfma_noalloc(const void* q, const void* k_cache, con
                                          const int32_t* block_table, const int32_t* tile_seq, const int32_t* tile_q0,
                                          const int32_t* tile_rows, const int32_t* positions, void* out, int64_t tokens,
                                          int n_tiles, int tile_queries, int n_splits, int heads, int kv_heads,
-                                         int head_dim, int page_size, int max_blocks, float scale, int window,
+                                         int head_dim, int page_size, int max_blocks, float scale, int span,
                                          int prefetch, int grouped, hipStream_t stream) {
   IX_REQUIRE(tokens >= 0 && heads > 0 && head_dim > 0 && n_splits >= 1 && n_splits <= 256, "sizes must be positive");
   float* part_o = nullptr;
@@ -558,5 +566,5 @@ extern "C" int ix_attention_mfma_noalloc(const void* q, const void* k_cache, con
   }
   return ix_attention_mfma(q, k_cache, v_cache, block_table, tile_seq, tile_q0, tile_rows, positions, out, part_o,
                            part_ml, tokens, n_tiles, tile_queries, n_splits, heads, kv_heads, head_dim, page_size,
-                           max_blocks, scale, window, prefetch, grouped, stream);
+                           max_blocks, scale, span, prefetch, grouped, stream);
 }

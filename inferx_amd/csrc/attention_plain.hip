@@ -6,7 +6,8 @@
 //
 // A query at position p reads keys [start, p], start = 0 or, with a window W,
 // max(0, p + 1 - W) (reference: PagedAttentionWithLseKernel, layers.cu:329-407;
-// window rule :346-354).  Query head h reads kv head h / (heads / kv_heads).
+// window rule :346-354) or, in chunks of C positions, p - p % C (`span`: see
+// ix_first_key in common.h).  Query head h reads kv head h / (heads / kv_heads).
 // Key j of a request lives in page table[j / page_size] at offset j % page_size;
 // keys are stored [page][kv_head][offset][d], values [page][kv_head][d][offset].
 // Values may be of another size than keys (`value_dim`).  `sink` (one float per head, or null): the softmax's
@@ -24,7 +25,7 @@ __global__ void __launch_bounds__(ATTN_PLAIN_THREADS)
 attn_plain_kernel(const T* __restrict__ q, const T* __restrict__ k_cache, const T* __restrict__ v_cache,
                   const int32_t* __restrict__ block_table, const int32_t* __restrict__ seq_of_token,
                   const int32_t* __restrict__ positions, T* __restrict__ out, int heads, int kv_heads, int head_dim,
-                  int value_dim, int page_size, int max_blocks, float scale, int window,
+                  int value_dim, int page_size, int max_blocks, float scale, int span,
                   const float* __restrict__ sink, const float2* __restrict__ turn_back, float softcap) {
   __shared__ float qs[256];
   __shared__ float sc[ATTN_PLAIN_THREADS];
@@ -37,7 +38,7 @@ attn_plain_kernel(const T* __restrict__ q, const T* __restrict__ k_cache, const 
   const int tid = threadIdx.x;
   const int64_t seq = seq_of_token[t];
   const int pos = positions[t];
-  const int start = (window > 0 && pos + 1 > window) ? pos + 1 - window : 0;
+  const int start = ix_first_key(pos, span);
   const int32_t* table = block_table + seq * max_blocks;
 
   if (tid < head_dim) qs[tid] = ix_load(q + (t * heads + head) * head_dim + tid);
@@ -95,24 +96,23 @@ attn_plain_kernel(const T* __restrict__ q, const T* __restrict__ k_cache, const 
 extern "C" int ix_attention_plain(const void* q, const void* k_cache, const void* v_cache, int dtype,
                                   const int32_t* block_table, const int32_t* seq_of_token, const int32_t* positions,
                                   void* out, int64_t tokens, int heads, int kv_heads, int head_dim, int value_dim,
-                                  int page_size, int max_blocks, float scale, int window, const float* sink,
+                                  int page_size, int max_blocks, float scale, int span, const float* sink,
                                   const float* turn_back, float softcap, hipStream_t stream) {
   IX_REQUIRE(tokens >= 0 && heads > 0 && kv_heads > 0 && page_size > 0 && max_blocks > 0, "sizes must be positive");
   IX_REQUIRE(heads % kv_heads == 0, "heads must be a multiple of kv_heads");
   IX_REQUIRE(head_dim > 0 && head_dim <= 256, "head_dim must be between 1 and 256");
   IX_REQUIRE(value_dim > 0 && value_dim <= 256, "value_dim must be between 1 and 256");
-  IX_REQUIRE(window >= 0, "window must not be negative");
   IX_REQUIRE(softcap >= 0.f, "the cap of the scores must not be negative");
   if (tokens == 0) return 0;
   dim3 grid(tokens, heads), block(ATTN_PLAIN_THREADS);
   if (dtype == IX_F32)
     hipLaunchKernelGGL(attn_plain_kernel<float>, grid, block, 0, stream, (const float*)q, (const float*)k_cache,
                        (const float*)v_cache, block_table, seq_of_token, positions, (float*)out, heads, kv_heads,
-                       head_dim, value_dim, page_size, max_blocks, scale, window, sink, (const float2*)turn_back, softcap);
+                       head_dim, value_dim, page_size, max_blocks, scale, span, sink, (const float2*)turn_back, softcap);
   else if (dtype == IX_BF16)
     hipLaunchKernelGGL(attn_plain_kernel<bf16_t>, grid, block, 0, stream, (const bf16_t*)q, (const bf16_t*)k_cache,
                        (const bf16_t*)v_cache, block_table, seq_of_token, positions, (bf16_t*)out, heads, kv_heads,
-                       head_dim, value_dim, page_size, max_blocks, scale, window, sink, (const float2*)turn_back, softcap);
+                       head_dim, value_dim, page_size, max_blocks, scale, span, sink, (const float2*)turn_back, softcap);
   else
     IX_REQUIRE(false, "dtype must be float32 or bfloat16");
   return ix_check_launch("ix_attention_plain");

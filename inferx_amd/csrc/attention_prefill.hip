@@ -33,7 +33,7 @@ attn_prefill_kernel(const __bf16* __restrict__ q, const __bf16* __restrict__ k_c
                     const int32_t* __restrict__ pair_b, const int32_t* __restrict__ positions,
                     __bf16* __restrict__ out, float* __restrict__ part_o, float* __restrict__ part_ml, int n_splits,
                     int heads, int kv_heads, int page_size, int max_blocks, float scale_log2,
-                    int window, int page_shift) {
+                    int span, int page_shift) {
   constexpr int D = 16 * NB;
   constexpr int NC = (NB + 1) / 2;          // 32-wide chunks of the head dimension
   constexpr int KS = 128;                   // elements per LDS row of the key tile: sixteen 16-byte pieces,
@@ -61,7 +61,7 @@ attn_prefill_kernel(const __bf16* __restrict__ q, const __bf16* __restrict__ k_c
   const int rows = tile_rows[tile];
   const int pos0 = positions[tq0];
   const int32_t* table = block_table + static_cast<int64_t>(tile_seq[tile]) * max_blocks;
-  const int lo = (window > 0 && pos0 + 1 > window) ? pos0 + 1 - window : 0;
+  const int lo = ix_first_key(pos0, span);
   // this workgroup's keys [kb0, hi): all that the tile reads, or one slice of them.  Slices are whole rounds of 64
   // keys from the tile's first round on, so a slice ends at a round's edge or where the tile's keys end, and the
   // masks below need not know of it.  A slice may be empty: then nothing is summed, and (-inf, 0, 0) is written.
@@ -74,6 +74,12 @@ attn_prefill_kernel(const __bf16* __restrict__ q, const __bf16* __restrict__ k_c
     hi = min(hi_tile, kb0 + per);
   }
   const int wq0 = 16 * QT * wave;  // this wavefront's first query within the tile
+  int first[QT], last_first[QT];  // the first key that this lane's query reads, and the last query of the sixteen
+#pragma unroll
+  for (int t = 0; t < QT; ++t) {
+    first[t] = ix_first_key(pos0 + wq0 + 16 * t + n, span);
+    last_first[t] = ix_first_key(pos0 + wq0 + 16 * t + 15, span);
+  }
 
   bf16x8 qf[QT][NC];
 #pragma unroll
@@ -251,13 +257,13 @@ attn_prefill_kernel(const __bf16* __restrict__ q, const __bf16* __restrict__ k_c
         }
         const int my_pos = pos0 + wq0 + 16 * t + n;
         const bool my_row = wq0 + 16 * t + n < rows;
-        const int my_lo = (window > 0 && my_pos + 1 > window) ? my_pos + 1 - window : 0;
+        const int my_lo = first[t];
         // scores stay unscaled: the scale (times log2 e) enters with the running maximum in one fused multiply-add
         float sv[8];
         float mx = -INFINITY;
         // keys that every query of these sixteen sees need no mask (uniform over the wavefront)
         const bool inner = wq0 + 16 * t + 16 <= rows && kb2 + 31 <= pos0 + wq0 + 16 * t &&
-                           (window == 0 || kb2 > pos0 + wq0 + 16 * t + 15 - window);
+                           kb2 >= last_first[t];
         if (inner) {
 #pragma unroll
           for (int j = 0; j < 8; ++j) {
@@ -341,13 +347,13 @@ static void launch_prefill(int tile_queries, dim3 grid, hipStream_t stream, cons
                            const void* v, const int32_t* table, const int32_t* tile_seq, const int32_t* tile_q0,
                            const int32_t* tile_rows, const int32_t* pair_a, const int32_t* pair_b,
                            const int32_t* positions, void* out, float* part_o, float* part_ml, int n_splits,
-                           int heads, int kv_heads, int page_size, int max_blocks, float scale_log2, int window) {
+                           int heads, int kv_heads, int page_size, int max_blocks, float scale_log2, int span) {
   int page_shift = 4;  // log2 of the page size, a power of two (the entry point has checked)
   while ((1 << page_shift) < page_size) ++page_shift;
   (void)tile_queries;  // 64: the entry point has checked
   hipLaunchKernelGGL((attn_prefill_kernel<NB, 1>), grid, dim3(256), 0, stream, (const __bf16*)q, (const __bf16*)k,
                      (const __bf16*)v, table, tile_seq, tile_q0, tile_rows, pair_a, pair_b, positions, (__bf16*)out, part_o,
-                     part_ml, n_splits, heads, kv_heads, page_size, max_blocks, scale_log2, window, page_shift);
+                     part_ml, n_splits, heads, kv_heads, page_size, max_blocks, scale_log2, span, page_shift);
 }
 
 // Tiles of up to `tile_queries` (64) consecutive queries of one request; head_dim a multiple of 16 up to 128; pages
@@ -363,13 +369,12 @@ extern "C" int ix_attention_prefill(const void* q, const void* k_cache, const vo
                                     int n_pairs, const int32_t* positions, void* out, float* part_o,
                                     float* part_ml, int n_splits, int64_t tokens, int n_tiles,
                                     int tile_queries, int heads, int kv_heads, int head_dim, int page_size,
-                                    int max_blocks, float scale, int window, hipStream_t stream) {
+                                    int max_blocks, float scale, int span, hipStream_t stream) {
   IX_REQUIRE(n_tiles >= 0 && heads > 0 && kv_heads > 0 && max_blocks > 0, "sizes must be positive");
   IX_REQUIRE(heads % kv_heads == 0, "heads must be a multiple of kv_heads");
   IX_REQUIRE(head_dim % 16 == 0 && head_dim >= 16 && head_dim <= 128, "head_dim must be a multiple of 16 up to 128");
   IX_REQUIRE(page_size >= 16 && (page_size & (page_size - 1)) == 0, "page_size must be a power of two from 16 on");
   IX_REQUIRE(tile_queries == 64, "a query tile holds up to 64 queries");
-  IX_REQUIRE(window >= 0, "window must not be negative");
   IX_REQUIRE(heads <= 65535, "too many heads");
   IX_REQUIRE(n_splits >= 1 && n_splits <= 256, "n_splits must be between 1 and 256");
   IX_REQUIRE(n_splits == 1 || (part_o != nullptr && part_ml != nullptr && tokens > 0), "workspace needed for split keys");
@@ -381,7 +386,7 @@ extern "C" int ix_attention_prefill(const void* q, const void* k_cache, const vo
   case NB:                                                                                                         \
     launch_prefill<NB>(tile_queries, grid, stream, q, k_cache, v_cache, block_table, tile_seq, tile_q0, tile_rows, \
                        pair_a, pair_b, positions, out, part_o, part_ml, n_splits, heads, kv_heads, page_size, max_blocks,  \
-                       scale_log2, window);                                                                        \
+                       scale_log2, span);                                                                        \
     break;
   switch (head_dim / 16) { CASE(1) CASE(2) CASE(3) CASE(4) CASE(5) CASE(6) CASE(7) CASE(8) }
 #undef CASE

@@ -55,7 +55,7 @@ attn_prefill128_kernel(const __bf16* __restrict__ q, const __bf16* k_cache, cons
                        const int32_t* __restrict__ pair_a, const int32_t* __restrict__ pair_b,
                        const int32_t* __restrict__ positions, __bf16* __restrict__ out, float* __restrict__ part_o,
                        float* __restrict__ part_ml, int n_splits, int heads, int kv_heads, int page_size,
-                       int max_blocks, float scale_log2, int window, int page_shift, const float* __restrict__ sink,
+                       int max_blocks, float scale_log2, int span, int page_shift, const float* __restrict__ sink,
                        float cap_slope, float cap2, const __bf16* __restrict__ gate, int64_t gate_stride) {
   constexpr int D = 32 * NB2;
   constexpr int NS = D / 16;                          // steps of 16 of the head dimension in K Q^T
@@ -89,7 +89,7 @@ attn_prefill128_kernel(const __bf16* __restrict__ q, const __bf16* k_cache, cons
     const int rows = tile_rows[tile];
     const int pos0 = positions[tq0];
     const int32_t* table = block_table + static_cast<int64_t>(tile_seq[tile]) * max_blocks;
-    const int lo = (window > 0 && pos0 + 1 > window) ? pos0 + 1 - window : 0;
+    const int lo = ix_first_key(pos0, span);
     // this workgroup's keys [kb0, hi): all that the tile reads, or one slice of them (whole rounds from the tile's
     // first round on; a slice may be empty: then (-inf, 0, 0) is written)
     const int hi_tile = pos0 + rows;
@@ -239,10 +239,11 @@ attn_prefill128_kernel(const __bf16* __restrict__ q, const __bf16* k_cache, cons
     const bool active = wq0 < rows;
     const int wfirst = pos0 + wq0;                  // position of its first query and of its last one
     const int wlast = pos0 + min(wq0 + 32, rows) - 1;
-    const int wlo = (window > 0 && wfirst + 1 > window) ? wfirst + 1 - window : 0;  // the first key any of them reads
+    const int wlo = ix_first_key(wfirst, span);  // the first key any of them reads
     const int my_pos = wfirst + qn;
     const bool my_row = wq0 + qn < rows;
-    const int my_lo = (window > 0 && my_pos + 1 > window) ? my_pos + 1 - window : 0;
+    const int my_lo = ix_first_key(my_pos, span);
+    const int wlast_lo = ix_first_key(wlast, span);  // from this key on no query of the wavefront skips one
 
     bf16x8 qf[NS];  // B operand of K Q^T: column qn, reduction indices 16 s + 8 h + j
 #pragma unroll
@@ -308,7 +309,7 @@ attn_prefill128_kernel(const __bf16* __restrict__ q, const __bf16* k_cache, cons
         __builtin_amdgcn_sched_barrier(0);
         // this lane: query qn, keys kb + 32 b + 8 c + 4 h + e for element 4 c + e of s[b]
         // keys that every query of the wavefront sees need no mask (uniform)
-        const bool inner = wq0 + 32 <= rows && kb + PW_KEYS - 1 <= wfirst && (window == 0 || kb > wlast - window);
+        const bool inner = wq0 + 32 <= rows && kb + PW_KEYS - 1 <= wfirst && kb >= wlast_lo;
         float mx = -INFINITY;
         const float sl = CAP ? 1.0f : scale_log2;  // (capped scores are in units of log2 already)
         if constexpr (CAP) {
@@ -423,7 +424,7 @@ extern "C" int ix_attention_prefill128(const void* q, const void* k_cache, const
                                        int n_pairs, const int32_t* positions, void* out, float* part_o,
                                        float* part_ml, int n_splits, int64_t tokens, int n_tiles, int heads,
                                        int kv_heads, int head_dim, int page_size, int max_blocks, float scale,
-                                       int window, const float* sink, float softcap, const void* gate,
+                                       int span, const float* sink, float softcap, const void* gate,
                                        int64_t gate_stride, hipStream_t stream) {
   IX_REQUIRE(softcap >= 0.f, "the cap of the scores must not be negative");
   IX_REQUIRE(gate == nullptr || gate_stride % 4 == 0, "a gate's rows must lie on 8-byte boundaries");
@@ -431,7 +432,6 @@ extern "C" int ix_attention_prefill128(const void* q, const void* k_cache, const
   IX_REQUIRE(heads % kv_heads == 0, "heads must be a multiple of kv_heads");
   IX_REQUIRE(head_dim % 32 == 0 && head_dim >= 32 && head_dim <= 128, "head_dim must be a multiple of 32 up to 128");
   IX_REQUIRE(page_size >= 16 && (page_size & (page_size - 1)) == 0, "page_size must be a power of two from 16 on");
-  IX_REQUIRE(window >= 0, "window must not be negative");
   IX_REQUIRE(n_splits >= 1 && n_splits <= 256, "n_splits must be between 1 and 256");
   IX_REQUIRE(n_splits == 1 || (part_o != nullptr && part_ml != nullptr && tokens > 0), "workspace needed for split keys");
   IX_REQUIRE(n_pairs >= 0 && n_pairs <= static_cast<int64_t>(n_tiles) * n_splits, "there are at most as many pairs as units");
@@ -446,7 +446,7 @@ extern "C" int ix_attention_prefill128(const void* q, const void* k_cache, const
   hipLaunchKernelGGL((attn_prefill128_kernel<NB2, CAP>), grid, dim3(512), 0, stream, (const __bf16*)q,               \
                      (const __bf16*)k_cache, (const __bf16*)v_cache, block_table, tile_seq, tile_q0, tile_rows,      \
                      pair_a, pair_b, positions, (__bf16*)out, part_o, part_ml, n_splits, heads, kv_heads, page_size, \
-                     max_blocks, scale_log2, window, page_shift, sink, cap_slope, cap2, (const __bf16*)gate, gate_stride)
+                     max_blocks, scale_log2, span, page_shift, sink, cap_slope, cap2, (const __bf16*)gate, gate_stride)
 #define CASE(NB2)                           \
   case NB2:                                 \
     if (softcap > 0.f) RUN(NB2, true);      \

@@ -120,9 +120,11 @@ __device__ __forceinline__ float ix_block_max(float v, float* red) {
   return total;
 }
 
-// What a gated product makes of its two sums g and u.  limit <= 0: silu(g) * u.  limit > 0, the clamped form:
-// g = min(g, limit), u = clamp(u, -limit, limit), then g * sigmoid(1.702 g) * (u + 1).
+// What a gated product makes of its two sums g and u.  limit 0: silu(g) * u.  limit > 0, the clamped form:
+// g = min(g, limit), u = clamp(u, -limit, limit), then g * sigmoid(1.702 g) * (u + 1).  limit < 0 (IX_GLU_GELU_TANH):
+// gelu(g) * u in gelu's tanh form, g / 2 (1 + tanh(y)) = g sigmoid(2 y) with y = sqrt(2 / pi) (g + 0.044715 g^3).
 #define IX_GLU_ALPHA 1.702f
+#define IX_GLU_GELU_TANH (-1.0f)
 template <bool FAST = false>
 __device__ __forceinline__ float ix_glu(float g, float u, float limit) {
   float steep = 1.0f;
@@ -130,9 +132,19 @@ __device__ __forceinline__ float ix_glu(float g, float u, float limit) {
     g = fminf(g, limit);
     u = fminf(fmaxf(u, -limit), limit) + 1.0f;
     steep = IX_GLU_ALPHA;
+  } else if (limit < 0.f) {
+    steep = 1.5957691216057308f * fmaf(0.044715f * g, g, 1.0f);  // 2 sqrt(2 / pi) (1 + 0.044715 g^2)
   }
   const float e = FAST ? __expf(-steep * g) : expf(-steep * g);
   return g / (1.0f + e) * u;
+}
+
+// The first key that a query at position `pos` reads, by how far its attention looks back: `span` 0 every earlier
+// position, W > 0 the last W (its own included), -C < 0 those of its own chunk, where a sequence falls into chunks of C
+// positions counted from 0.  It never decreases with the position.
+__device__ __forceinline__ int ix_first_key(int pos, int span) {
+  if (span > 0) return max(pos + 1 - span, 0);
+  return span < 0 ? pos - pos % -span : 0;
 }
 
 // A score capped on its way into the softmax: c tanh(score / c), in units of log2 (c log2(e) = cap2), from the raw product
@@ -153,10 +165,11 @@ void ix_set_error(const std::string& msg);
 // out[t, h, :] from the parts that kernels which cut keys into slices leave (attention_mfma.hip)
 // (turn_back: float32 (cos, sin) [tokens, head_dim / 2]; the result is rotated by minus these angles, or null; gate:
 // bfloat16, token t's numbers for head h from gate + t * gate_stride + h * head_dim on; the result is multiplied by
-// their sigmoid, or null)
+// their sigmoid, or null; head_gate: bfloat16, one number per head from head_gate + t * head_gate_stride on, likewise)
 int ix_attention_combine(const float* part_o, const float* part_ml, void* out, int64_t tokens, int heads,
                          int n_splits, int head_dim, hipStream_t stream, const float* turn_back = nullptr,
-                         const void* gate = nullptr, int64_t gate_stride = 0);
+                         const void* gate = nullptr, int64_t gate_stride = 0, const void* head_gate = nullptr,
+                         int64_t head_gate_stride = 0);
 int ix_check_launch(const char* what);
 #define IX_REQUIRE(cond, msg)                          \
   do {                                                 \

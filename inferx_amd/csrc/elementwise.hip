@@ -560,7 +560,7 @@ extern "C" int ix_qkv_rope_append(const void* qkv, int dtype, const void* bias, 
 
 // ---------------------------------------------------------------------------
 // out[t, i] = glu(gu[t, i] + bias[i], gu[t, width + i] + bias[width + i]) with `ix_glu` (silu(g) * u, or with a
-// limit the clamped form); the bias (2 * width numbers, gate's first) may be absent.
+// limit another form); the bias (2 * width numbers, gate's first) may be absent.
 template <typename T>
 __global__ void glu_bias_kernel(const T* __restrict__ gu, const void* __restrict__ bias, int bias_dtype,
                                 T* __restrict__ out, int64_t tokens, int64_t width, float limit) {
@@ -578,6 +578,41 @@ __global__ void glu_bias_kernel(const T* __restrict__ gu, const void* __restrict
   }
 }
 
+// bfloat16 with a width that is a multiple of 8: eight numbers per thread, 16-byte loads and stores
+__global__ void __launch_bounds__(256)
+glu_bias_vec8_kernel(const uint16_t* __restrict__ gu, const void* __restrict__ bias, int bias_dtype,
+                     uint16_t* __restrict__ out, int64_t tokens, int64_t width, float limit) {
+  const int64_t per_row = width / 8, n = tokens * per_row;
+  for (int64_t p = static_cast<int64_t>(blockIdx.x) * blockDim.x + threadIdx.x; p < n;
+       p += static_cast<int64_t>(gridDim.x) * blockDim.x) {
+    const int64_t t = p / per_row, c = (p - t * per_row) * 8;
+    const uint4 g4 = *reinterpret_cast<const uint4*>(gu + t * 2 * width + c);
+    const uint4 u4 = *reinterpret_cast<const uint4*>(gu + t * 2 * width + width + c);
+    const uint32_t gw[4] = {g4.x, g4.y, g4.z, g4.w}, uw[4] = {u4.x, u4.y, u4.z, u4.w};
+    float g[8], u[8];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      g[2 * i] = __uint_as_float(gw[i] << 16);
+      g[2 * i + 1] = __uint_as_float(gw[i] & 0xffff0000u);
+      u[2 * i] = __uint_as_float(uw[i] << 16);
+      u[2 * i + 1] = __uint_as_float(uw[i] & 0xffff0000u);
+    }
+    if (bias) {
+#pragma unroll
+      for (int i = 0; i < 8; ++i) {
+        g[i] += ix_load_rt(bias, bias_dtype, c + i);
+        u[i] += ix_load_rt(bias, bias_dtype, width + c + i);
+      }
+    }
+    uint32_t o[4];
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+      o[i] = ix_f32_to_bf16(ix_glu<true>(g[2 * i], u[2 * i], limit)) |
+             static_cast<uint32_t>(ix_f32_to_bf16(ix_glu<true>(g[2 * i + 1], u[2 * i + 1], limit))) << 16;
+    *reinterpret_cast<uint4*>(out + t * width + c) = make_uint4(o[0], o[1], o[2], o[3]);
+  }
+}
+
 extern "C" int ix_glu_bias(const void* gu, const void* bias, int bias_dtype, void* out, int dtype, int64_t tokens,
                            int64_t width, float limit, hipStream_t stream) {
   IX_REQUIRE(tokens >= 0 && width > 0, "sizes must be positive");
@@ -587,6 +622,10 @@ extern "C" int ix_glu_bias(const void* gu, const void* bias, int bias_dtype, voi
   if (dtype == IX_F32)
     hipLaunchKernelGGL(glu_bias_kernel<float>, grid, block, 0, stream, (const float*)gu, bias, bias_dtype,
                        (float*)out, tokens, width, limit);
+  else if (dtype == IX_BF16 && width % 8 == 0 &&
+           ((reinterpret_cast<uintptr_t>(gu) | reinterpret_cast<uintptr_t>(out)) & 15) == 0)
+    hipLaunchKernelGGL(glu_bias_vec8_kernel, dim3(static_cast<unsigned>(std::min<int64_t>((n / 8 + 255) / 256, 65536))),
+                       block, 0, stream, (const uint16_t*)gu, bias, bias_dtype, (uint16_t*)out, tokens, width, limit);
   else if (dtype == IX_BF16)
     hipLaunchKernelGGL(glu_bias_kernel<bf16_t>, grid, block, 0, stream, (const bf16_t*)gu, bias, bias_dtype,
                        (bf16_t*)out, tokens, width, limit);
@@ -594,39 +633,6 @@ extern "C" int ix_glu_bias(const void* gu, const void* bias, int bias_dtype, voi
     IX_REQUIRE(false, "dtype must be float32 or bfloat16");
   return ix_check_launch("ix_glu_bias");
 }
-
-// ---------------------------------------------------------------------------
-// h[t, c] += a[t, c] + b[t, c] + bias[c]: two branches' results (the second and the bias may be absent) summed in
-// float32 and added to the float32 residual stream.
-template <typename T>
-__global__ void add_branches_kernel(float* __restrict__ h, const T* __restrict__ a, const T* __restrict__ b,
-                                    const void* __restrict__ bias, int bias_dtype, int64_t n, int64_t width) {
-  for (int64_t i = static_cast<int64_t>(blockIdx.x) * blockDim.x + threadIdx.x; i < n;
-       i += static_cast<int64_t>(gridDim.x) * blockDim.x) {
-    float d = ix_load(a + i);
-    if (b) d += ix_load(b + i);
-    if (bias) d += ix_load_rt(bias, bias_dtype, i % width);
-    h[i] += d;
-  }
-}
-
-extern "C" int ix_add_branches(float* h, const void* a, const void* b, int dtype, const void* bias, int bias_dtype,
-                               int64_t tokens, int64_t width, hipStream_t stream) {
-  IX_REQUIRE(tokens >= 0 && width > 0, "sizes must be positive");
-  if (tokens == 0) return 0;
-  const int64_t n = tokens * width;
-  dim3 grid(static_cast<unsigned>(std::min<int64_t>((n + 255) / 256, 65536))), block(256);
-  if (dtype == IX_F32)
-    hipLaunchKernelGGL(add_branches_kernel<float>, grid, block, 0, stream, h, (const float*)a, (const float*)b, bias,
-                       bias_dtype, n, width);
-  else if (dtype == IX_BF16)
-    hipLaunchKernelGGL(add_branches_kernel<bf16_t>, grid, block, 0, stream, h, (const bf16_t*)a, (const bf16_t*)b,
-                       bias, bias_dtype, n, width);
-  else
-    IX_REQUIRE(false, "dtype must be float32 or bfloat16");
-  return ix_check_launch("ix_add_branches");
-}
-
 
 // ---------------------------------------------------------------------------
 // The PolyNorm activation, a workgroup per row:

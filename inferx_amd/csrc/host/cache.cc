@@ -49,7 +49,7 @@ struct Request {
 };
 
 struct Cache {
-  std::vector<int32_t> windows;
+  std::vector<int32_t> windows;  // per group: 0 keeps every token, W > 0 the last W, -C < 0 those of the current chunk of C
   std::vector<int32_t> keeps;  // per group: the first tokens of a request that a windowed group never gives back
   std::vector<Pool> pools;
   int32_t page_size = 0, max_requests = 0, max_blocks = 0;
@@ -70,8 +70,8 @@ struct Cache {
   }
   int64_t first_live_page(size_t g, int64_t cached) const {
     const int64_t w = windows[g];
-    if (w <= 0) return 0;
-    const int64_t start = cached + 1 - w;
+    if (w == 0) return 0;
+    const int64_t start = w > 0 ? cached + 1 - w : cached - cached % -w;
     return (start > 0 ? start : 0) / page_size;
   }
   bool release_page(size_t g, int32_t page) {
@@ -106,12 +106,12 @@ struct Cache {
     return ok;
   }
   // Pages of group g that a request which has `cached` tokens and a reservation up to `upto` holds now.  A group
-  // that keeps every token holds all of them.  A windowed group, when the largest step is known (step_cap), holds
+  // that keeps every token holds all of them.  A windowed or chunked group, when the largest step is known (step_cap), holds
   // only what the next step can touch, cached + step_cap tokens at most: its pages beyond that are taken when the
   // steps get there (its pool is sized so that they are there, see pages_for_window in cache/manager.py), so
   // that a long prompt does not claim a context's worth of pages in a group that only ever reads a window.
   int64_t pages_held(size_t g, int64_t cached, int64_t upto) const {
-    if (windows[g] > 0 && step_cap > 0 && upto > cached + step_cap) upto = cached + step_cap;
+    if (windows[g] != 0 && step_cap > 0 && upto > cached + step_cap) upto = cached + step_cap;
     return (upto + page_size - 1) / page_size;
   }
   // 0 ok, 1 pool empty, 2 context full, -1 error

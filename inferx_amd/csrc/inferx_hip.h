@@ -21,13 +21,14 @@ int ix_abi_version();
 //   block_table   int32 [requests, max_blocks]
 //   tile_seq / tile_q0 / tile_rows   int32 [n_tiles]: request, first token row, rows (<= tile_queries) of a tile
 //   positions     int32 [tokens]
+//   span          how far back a query reads: 0 every earlier position, W > 0 the last W, -C < 0 its own chunk of C
 //   part_o        float32 [tokens * heads * n_splits * head_dim], part_ml float32 [tokens * heads * n_splits * 2]:
 //                 the slices' partial results, needed when n_splits > 1 (the caller's workspace)
 int ix_attention_mfma(const void* q, const void* k_cache, const void* v_cache, const int32_t* block_table,
                       const int32_t* tile_seq, const int32_t* tile_q0, const int32_t* tile_rows,
                       const int32_t* positions, void* out, float* part_o, float* part_ml, int64_t tokens, int n_tiles,
                       int tile_queries, int n_splits, int heads, int kv_heads, int head_dim, int page_size,
-                      int max_blocks, float scale, int window, int prefetch, int grouped, hipStream_t stream);
+                      int max_blocks, float scale, int span, int prefetch, int grouped, hipStream_t stream);
 
 // The same operation for callers that cannot allocate device memory: code under HIP graph capture, tight
 // serving loops that must not call hipMalloc, harnesses that forbid it.  It has no counterpart in the reference,
@@ -50,7 +51,7 @@ int ix_attention_mfma_noalloc(const void* q, const void* k_cache, const void* v_
                               const int32_t* tile_seq, const int32_t* tile_q0, const int32_t* tile_rows,
                               const int32_t* positions, void* out, int64_t tokens, int n_tiles, int tile_queries,
                               int n_splits, int heads, int kv_heads, int head_dim, int page_size, int max_blocks,
-                              float scale, int window, int prefetch, int grouped, hipStream_t stream);
+                              float scale, int span, int prefetch, int grouped, hipStream_t stream);
 
 #ifdef __cplusplus
 }

@@ -102,6 +102,7 @@ extern "C" int ix_latent_prepare(void* q, int64_t q_stride, const void* dkv, int
 //   ql   element (t, h, i) at ql[t * ql_t + h * ql_h + i], i < rank       (the query moved to the latent's side)
 //   qr   element (t, h, i) at qr[t * qr_t + h * qr_h + i], i < rot_dim    (its rotated part)
 //   out  element (t, h, i) at out[t * out_t + h * out_h + i], i < rank
+//   head_gate (or null): the result of (t, h) is multiplied by the sigmoid of head_gate[t * gate_stride + h]
 #define LAT_THREADS 256
 #define LAT_MAX_WIDTH 1088
 #define LAT_ACC 4
@@ -112,7 +113,7 @@ latent_attn_plain_kernel(const T* __restrict__ ql, int64_t ql_t, int64_t ql_h, c
                          int64_t qr_h, const T* __restrict__ cache, const int32_t* __restrict__ block_table,
                          const int32_t* __restrict__ seq_of_token, const int32_t* __restrict__ positions,
                          T* __restrict__ out, int64_t out_t, int64_t out_h, int rank, int rot_dim, int page_size,
-                         int max_blocks, float scale, int window) {
+                         int max_blocks, float scale, int window, const T* __restrict__ head_gate, int64_t gate_stride) {
   __shared__ float qs[LAT_MAX_WIDTH];
   __shared__ float sc[LAT_THREADS];
   __shared__ int64_t at[LAT_THREADS];
@@ -161,6 +162,7 @@ latent_attn_plain_kernel(const T* __restrict__ ql, int64_t ql_t, int64_t ql_h, c
     }
     __syncthreads();
   }
+  if (head_gate) l *= 1.0f + expf(-ix_load(head_gate + t * gate_stride + head));
 #pragma unroll
   for (int a = 0; a < LAT_ACC; ++a) {
     const int c = tid + a * LAT_THREADS;
@@ -173,7 +175,7 @@ extern "C" int ix_latent_attention_plain(const void* ql, int64_t ql_t, int64_t q
                                          const int32_t* seq_of_token, const int32_t* positions, void* out,
                                          int64_t out_t, int64_t out_h, int64_t tokens, int heads, int rank,
                                          int rot_dim, int page_size, int max_blocks, float scale, int window,
-                                         hipStream_t stream) {
+                                         const void* head_gate, int64_t gate_stride, hipStream_t stream) {
   IX_REQUIRE(tokens >= 0 && heads > 0 && rank > 0 && rot_dim >= 0 && page_size > 0 && max_blocks > 0 && window >= 0,
              "sizes must be positive");
   IX_REQUIRE(rank <= LAT_ACC * LAT_THREADS && rank + rot_dim <= LAT_MAX_WIDTH,
@@ -184,11 +186,13 @@ extern "C" int ix_latent_attention_plain(const void* ql, int64_t ql_t, int64_t q
   if (dtype == IX_F32)
     hipLaunchKernelGGL(latent_attn_plain_kernel<float>, grid, block, 0, stream, (const float*)ql, ql_t, ql_h,
                        (const float*)qr, qr_t, qr_h, (const float*)cache, block_table, seq_of_token, positions,
-                       (float*)out, out_t, out_h, rank, rot_dim, page_size, max_blocks, scale, window);
+                       (float*)out, out_t, out_h, rank, rot_dim, page_size, max_blocks, scale, window,
+                       (const float*)head_gate, gate_stride);
   else if (dtype == IX_BF16)
     hipLaunchKernelGGL(latent_attn_plain_kernel<bf16_t>, grid, block, 0, stream, (const bf16_t*)ql, ql_t, ql_h,
                        (const bf16_t*)qr, qr_t, qr_h, (const bf16_t*)cache, block_table, seq_of_token, positions,
-                       (bf16_t*)out, out_t, out_h, rank, rot_dim, page_size, max_blocks, scale, window);
+                       (bf16_t*)out, out_t, out_h, rank, rot_dim, page_size, max_blocks, scale, window,
+                       (const bf16_t*)head_gate, gate_stride);
   else
     IX_REQUIRE(false, "dtype must be float32 or bfloat16");
   return ix_check_launch("ix_latent_attention_plain");
@@ -229,7 +233,7 @@ latent_attn_mfma_kernel(const __bf16* __restrict__ ql, int64_t ql_t, int64_t ql_
                         const int32_t* __restrict__ positions, __bf16* __restrict__ out, int64_t out_t, int64_t out_h,
                         float* __restrict__ part_o, float* __restrict__ part_ml, int n_splits, int tokens, int heads,
                         int rank, int rot_dim, int page_size, int max_blocks, float scale_log2, int n_tiles,
-                        int window) {
+                        int window, const __bf16* __restrict__ head_gate, int64_t gate_stride) {
   extern __shared__ __attribute__((aligned(16))) unsigned char latm_lds[];
   constexpr int NP = (4 * NW + 7) / 8;  // 16-byte pieces of a round's rows that a thread moves
   const int width = rank + rot_dim;
@@ -412,7 +416,7 @@ latent_attn_mfma_kernel(const __bf16* __restrict__ ql, int64_t ql_t, int64_t ql_
       part_ml[2 * p + 1] = lt;
     }
   } else {
-    const float inv = 1.0f / lt;
+    const float inv = head_gate ? 1.0f / (lt * (1.0f + __expf(-(float)head_gate[row * gate_stride + head]))) : 1.0f / lt;
 #pragma unroll
     for (int d = 0; d < NR; ++d) {
       if (d < nr) {
@@ -427,13 +431,14 @@ latent_attn_mfma_kernel(const __bf16* __restrict__ ql, int64_t ql_t, int64_t ql_
 
 // decode != 0: one token per request (tokens == requests); with n_splits > 1 the keys are cut into that many slices,
 // part_o float32 [tokens * heads * n_splits, rank] and part_ml float32 [tokens * heads * n_splits, 2] take what the
-// slices leave, and out must be contiguous [tokens, heads, rank].
+// slices leave, and out must be contiguous [tokens, heads, rank].  head_gate as for the plain kernel (bfloat16).
 extern "C" int ix_latent_attention_mfma(const void* ql, int64_t ql_t, int64_t ql_h, const void* qr, int64_t qr_t,
                                         int64_t qr_h, const void* cache, const int32_t* block_table,
                                         const int32_t* seq_of_token, const int32_t* positions, void* out,
                                         int64_t out_t, int64_t out_h, float* part_o, float* part_ml, int n_splits,
                                         int64_t tokens, int heads, int rank, int rot_dim, int page_size,
-                                        int max_blocks, float scale, int decode, int window, hipStream_t stream) {
+                                        int max_blocks, float scale, int decode, int window, const void* head_gate,
+                                        int64_t gate_stride, hipStream_t stream) {
   IX_REQUIRE(tokens >= 0 && tokens < (1 << 30) && heads > 0 && rank > 0 && rot_dim >= 0 && page_size > 0 && max_blocks > 0 &&
                  window >= 0, "sizes must be positive");
   const int width = rank + rot_dim;
@@ -469,7 +474,7 @@ extern "C" int ix_latent_attention_mfma(const void* ql, int64_t ql_t, int64_t ql
     hipLaunchKernelGGL(kernel, grid, dim3(256), lds, stream, (const __bf16*)ql, ql_t, ql_h, (const __bf16*)qr, qr_t,     \
                        qr_h, (const __bf16*)cache, block_table, seq_of_token, positions, (__bf16*)out, out_t, out_h,     \
                        part_o, part_ml, n_splits, static_cast<int>(tokens), heads, rank, rot_dim, page_size, max_blocks, \
-                       scale_log2, n_tiles, window);                                                                    \
+                       scale_log2, n_tiles, window, (const __bf16*)head_gate, gate_stride);                              \
   } while (0)
 #define BY_SIZE(DEC)                                        \
   if (width <= 128 && rank <= 128) LAUNCH(4, 8, DEC);       \
@@ -479,6 +484,8 @@ extern "C" int ix_latent_attention_mfma(const void* ql, int64_t ql_t, int64_t ql
 #undef BY_SIZE
 #undef LAUNCH
   if (ix_check_launch("ix_latent_attention_mfma")) return 1;
-  if (n_splits > 1) return ix_attention_combine(part_o, part_ml, out, tokens, heads, n_splits, rank, stream);
+  if (n_splits > 1)
+    return ix_attention_combine(part_o, part_ml, out, tokens, heads, n_splits, rank, stream, nullptr, nullptr, 0, head_gate,
+                                gate_stride);
   return 0;
 }

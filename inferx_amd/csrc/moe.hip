@@ -103,8 +103,8 @@ __device__ __forceinline__ void route_select(float* z, float* red, float* __rest
 template <typename T>
 __global__ void __launch_bounds__(ROUTE_THREADS)
 moe_route_kernel(const T* __restrict__ x, const void* __restrict__ wr, int wr_dtype,
-                 const void* __restrict__ shared_gate_w, int sg_dtype, float* __restrict__ topk_w,
-                 int32_t* __restrict__ topk_e, float* __restrict__ shared_gate, int64_t width, int experts, int k,
+                 const void* __restrict__ shared_gate_w, int sg_dtype, const float* __restrict__ bias,
+                 float* __restrict__ topk_w, int32_t* __restrict__ topk_e, float* __restrict__ shared_gate, int64_t width, int experts, int k,
                  int renormalize, float scale, int always, int n_groups, int groups_keep) {
   extern __shared__ __align__(16) float smem[];
   float* xs = smem;                        // [width rounded up to 4]
@@ -119,7 +119,7 @@ moe_route_kernel(const T* __restrict__ x, const void* __restrict__ wr, int wr_dt
     const bool routed = e < experts;
     const float dot = route_row_dot(xs, routed ? wr : shared_gate_w, routed ? wr_dtype : sg_dtype,
                                     routed ? static_cast<int64_t>(e) * width : 0, width, lane);
-    if (lane == 0) z[e] = dot;
+    if (lane == 0) z[e] = dot + (bias && routed ? bias[e] : 0.f);
   }
   __syncthreads();
   const float gate = shared_gate_w ? 1.0f / (1.0f + expf(-z[experts])) : 1.0f;
@@ -132,8 +132,8 @@ moe_route_kernel(const T* __restrict__ x, const void* __restrict__ wr, int wr_dt
 template <typename T>
 __global__ void __launch_bounds__(ROUTE_THREADS)
 moe_route_logits_kernel(const T* __restrict__ x, const void* __restrict__ wr, int wr_dtype,
-                        const void* __restrict__ shared_gate_w, int sg_dtype, float* __restrict__ logits,
-                        int64_t width, int experts) {
+                        const void* __restrict__ shared_gate_w, int sg_dtype, const float* __restrict__ bias,
+                        float* __restrict__ logits, int64_t width, int experts) {
   extern __shared__ __align__(16) float xs[];  // [width]
   const int64_t t = blockIdx.x;
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
@@ -145,7 +145,7 @@ moe_route_logits_kernel(const T* __restrict__ x, const void* __restrict__ wr, in
   const bool routed = e < experts;
   const float dot = route_row_dot(xs, routed ? wr : shared_gate_w, routed ? wr_dtype : sg_dtype,
                                   routed ? static_cast<int64_t>(e) * width : 0, width, lane);
-  if (lane == 0) logits[t * (experts + 1) + e] = dot;
+  if (lane == 0) logits[t * (experts + 1) + e] = dot + (bias && routed ? bias[e] : 0.f);
 }
 
 __global__ void __launch_bounds__(64)
@@ -171,8 +171,8 @@ typedef __bf16 route_bf16x8 __attribute__((ext_vector_type(8)));
 typedef float route_f32x4 __attribute__((ext_vector_type(4)));
 __global__ void __launch_bounds__(256)
 moe_route_logits_mfma_kernel(const __bf16* __restrict__ x, const __bf16* __restrict__ wr,
-                             const __bf16* __restrict__ shared_gate_w, float* __restrict__ logits, int64_t tokens,
-                             int width, int experts) {
+                             const __bf16* __restrict__ shared_gate_w, const float* __restrict__ bias,
+                             float* __restrict__ logits, int64_t tokens, int width, int experts) {
   __shared__ route_f32x4 part[4][64];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int m = lane & 15, g = lane >> 4;
@@ -204,16 +204,19 @@ moe_route_logits_mfma_kernel(const __bf16* __restrict__ x, const __bf16* __restr
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
       const int row = 16 * blockIdx.y + 4 * g + i;
-      if (t < tokens && row < rows) logits[t * (experts + 1) + row] = sum[i];
+      if (t < tokens && row < rows)
+        logits[t * (experts + 1) + row] = sum[i] + (bias && row < experts ? bias[row] : 0.f);
     }
   }
 }
 
+// `bias` (float32 [experts], or null) is added to the experts' scores before anything else.
 // `logits_scratch`: float32 [tokens, experts + 1], used when tokens <= ROUTE_SMALL_TOKENS, and for more tokens when
 // activations and weights are bfloat16 (may be null: then one kernel per token computes and selects).
 #define ROUTE_SMALL_TOKENS 128
 extern "C" int ix_moe_route(const void* x, int dtype, const void* wr, int wr_dtype, const void* shared_gate_w,
-                            int sg_dtype, float* topk_w, int32_t* topk_e, float* shared_gate, float* logits_scratch,
+                            int sg_dtype, const float* bias, float* topk_w, int32_t* topk_e, float* shared_gate,
+                            float* logits_scratch,
                             int64_t tokens, int64_t width, int experts, int k, int renormalize, float scale,
                             int always, int n_groups, int groups_keep, hipStream_t stream) {
   IX_REQUIRE(tokens >= 0 && width > 0, "sizes must be positive");
@@ -234,10 +237,10 @@ extern "C" int ix_moe_route(const void* x, int dtype, const void* wr, int wr_dty
     const size_t xs_bytes = ((width + 3) & ~3) * sizeof(float);
     if (dtype == IX_F32)
       hipLaunchKernelGGL(moe_route_logits_kernel<float>, grid, block, xs_bytes, stream, (const float*)x, wr, wr_dtype,
-                         shared_gate_w, sg_dtype, logits_scratch, width, experts);
+                         shared_gate_w, sg_dtype, bias, logits_scratch, width, experts);
     else
       hipLaunchKernelGGL(moe_route_logits_kernel<bf16_t>, grid, block, xs_bytes, stream, (const bf16_t*)x, wr,
-                         wr_dtype, shared_gate_w, sg_dtype, logits_scratch, width, experts);
+                         wr_dtype, shared_gate_w, sg_dtype, bias, logits_scratch, width, experts);
     hipLaunchKernelGGL(moe_route_select_kernel, dim3(tokens), dim3(64), experts * sizeof(float), stream,
                        logits_scratch, topk_w, topk_e, shared_gate_w ? shared_gate : nullptr, experts, k, renormalize,
                        scale, always, n_groups, groups_keep);
@@ -248,7 +251,7 @@ extern "C" int ix_moe_route(const void* x, int dtype, const void* wr, int wr_dty
       ((reinterpret_cast<uintptr_t>(x) | reinterpret_cast<uintptr_t>(wr) | reinterpret_cast<uintptr_t>(shared_gate_w)) & 15) == 0) {
     const int row_blocks = (experts + (shared_gate_w ? 1 : 0) + 15) / 16;
     hipLaunchKernelGGL(moe_route_logits_mfma_kernel, dim3(static_cast<unsigned>((tokens + 15) / 16), row_blocks),
-                       dim3(256), 0, stream, (const __bf16*)x, (const __bf16*)wr, (const __bf16*)shared_gate_w, logits_scratch,
+                       dim3(256), 0, stream, (const __bf16*)x, (const __bf16*)wr, (const __bf16*)shared_gate_w, bias, logits_scratch,
                        tokens, (int)width, experts);
     hipLaunchKernelGGL(moe_route_select_kernel, dim3(tokens), dim3(64), experts * sizeof(float), stream,
                        logits_scratch, topk_w, topk_e, shared_gate_w ? shared_gate : nullptr, experts, k, renormalize,
@@ -258,11 +261,11 @@ extern "C" int ix_moe_route(const void* x, int dtype, const void* wr, int wr_dty
   dim3 grid(tokens), block(ROUTE_THREADS);
   if (dtype == IX_F32)
     hipLaunchKernelGGL(moe_route_kernel<float>, grid, block, smem, stream, (const float*)x, wr, wr_dtype,
-                       shared_gate_w, sg_dtype, topk_w, topk_e, shared_gate, width, experts, k, renormalize, scale,
+                       shared_gate_w, sg_dtype, bias, topk_w, topk_e, shared_gate, width, experts, k, renormalize, scale,
                        always, n_groups, groups_keep);
   else
     hipLaunchKernelGGL(moe_route_kernel<bf16_t>, grid, block, smem, stream, (const bf16_t*)x, wr, wr_dtype,
-                       shared_gate_w, sg_dtype, topk_w, topk_e, shared_gate, width, experts, k, renormalize, scale,
+                       shared_gate_w, sg_dtype, bias, topk_w, topk_e, shared_gate, width, experts, k, renormalize, scale,
                        always, n_groups, groups_keep);
   return ix_check_launch("ix_moe_route");
 }

@@ -26,7 +26,8 @@ __global__ void __launch_bounds__(RF_THREADS)
 moe_route_dispatch_small_kernel(const T* __restrict__ x, float* h, const T* __restrict__ delta,
                                 const void* __restrict__ gamma, int gamma_dtype, float eps, T* __restrict__ x_out,
                                 const void* __restrict__ wr, int wr_dtype,
-                                const void* __restrict__ shared_gate_w, int sg_dtype, float* logits,
+                                const void* __restrict__ shared_gate_w, int sg_dtype, const float* __restrict__ bias,
+                                float* logits,
                                 int32_t* arrived, int64_t width, float* __restrict__ topk_w,
                                 int32_t* __restrict__ topk_e, float* __restrict__ shared_gate,
                                 int32_t* __restrict__ offsets, int32_t* __restrict__ rows, int32_t* __restrict__ dest,
@@ -49,6 +50,7 @@ moe_route_dispatch_small_kernel(const T* __restrict__ x, float* h, const T* __re
   const bool preloaded = e < n_rows && route_row_preloadable(w_row, routed ? wr_dtype : sg_dtype, width);
   uint4 w_pre[ROUTE_PRELOAD];
   if (preloaded) route_row_preload(w_row, w_base, width, lane, w_pre);
+  const float bias_e = bias && routed ? bias[e] : 0.f;
   if (NORM) {
     const float* hr = h + t * width;
     const T* dr = delta + t * width;
@@ -87,7 +89,8 @@ moe_route_dispatch_small_kernel(const T* __restrict__ x, float* h, const T* __re
   if (e < n_rows) {
     const float dot = preloaded ? route_row_dot_preloaded(xs, w_row, w_base, width, lane, w_pre)
                                 : route_row_dot(xs, w_row, routed ? wr_dtype : sg_dtype, w_base, width, lane);
-    if (lane == 0) __hip_atomic_store(&logits[t * (experts + 1) + e], dot, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+    if (lane == 0)
+      __hip_atomic_store(&logits[t * (experts + 1) + e], dot + bias_e, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
   }
   __builtin_amdgcn_s_waitcnt(0);  // this wavefront's loads have arrived and its store has been acknowledged
   __syncthreads();
@@ -118,7 +121,8 @@ moe_route_dispatch_small_kernel(const T* __restrict__ x, float* h, const T* __re
 
 static int route_dispatch_small_launch(const void* x, float* h, const void* delta, const void* gamma, int gamma_dtype,
                                        float eps, void* x_out, int dtype, const void* wr, int wr_dtype,
-                                       const void* shared_gate_w, int sg_dtype, float* logits, int32_t* arrived,
+                                       const void* shared_gate_w, int sg_dtype, const float* bias, float* logits,
+                                       int32_t* arrived,
                                        int64_t width, float* topk_w, int32_t* topk_e, float* shared_gate,
                                        int32_t* offsets, int32_t* rows, int32_t* dest, int tokens, int experts,
                                        int k, int renormalize, float scale, int n_groups, int groups_keep, int tile_rows, int32_t* tile_expert,
@@ -141,7 +145,7 @@ static int route_dispatch_small_launch(const void* x, float* h, const void* delt
 #define LAUNCH(T, NORM)                                                                                             \
   hipLaunchKernelGGL((moe_route_dispatch_small_kernel<T, NORM>), grid, block, xs_bytes, stream, (const T*)x, h,     \
                      (const T*)delta, gamma, gamma_dtype, eps, (T*)x_out, wr, wr_dtype, shared_gate_w, sg_dtype,    \
-                     logits, arrived, width, topk_w, topk_e, shared_gate, offsets, rows, dest, tokens, experts, k,  \
+                     bias, logits, arrived, width, topk_w, topk_e, shared_gate, offsets, rows, dest, tokens, experts, k,  \
                      renormalize, scale, n_groups, groups_keep, tile_rows, tile_expert, tile_row0, tile_info)
   if (h) {
     if (dtype == IX_F32) LAUNCH(float, true);
@@ -156,16 +160,17 @@ static int route_dispatch_small_launch(const void* x, float* h, const void* delt
 
 // x [tokens <= 16, width]; logits float32 [tokens, experts + 1] (scratch); arrived: 17 int32 (one for the launch, one
 // per token), zero, left zero.
-// Calls that share `arrived` must not overlap.
+// `bias` (float32 [experts], or null) is added to the experts' scores.  Calls that share `arrived` must not overlap.
 extern "C" int ix_moe_route_dispatch_small(const void* x, int dtype, const void* wr, int wr_dtype,
-                                           const void* shared_gate_w, int sg_dtype, float* logits, int32_t* arrived,
+                                           const void* shared_gate_w, int sg_dtype, const float* bias, float* logits,
+                                           int32_t* arrived,
                                            int64_t width, float* topk_w, int32_t* topk_e, float* shared_gate,
                                            int32_t* offsets, int32_t* rows, int32_t* dest, int tokens, int experts,
                                            int k, int renormalize, float scale, int n_groups, int groups_keep, int tile_rows, int32_t* tile_expert,
                                            int32_t* tile_row0, int32_t* tile_info, hipStream_t stream) {
   IX_REQUIRE(x != nullptr, "x needed");
   return route_dispatch_small_launch(x, nullptr, nullptr, nullptr, IX_F32, 0.f, nullptr, dtype, wr, wr_dtype,
-                                     shared_gate_w, sg_dtype, logits, arrived, width, topk_w, topk_e, shared_gate,
+                                     shared_gate_w, sg_dtype, bias, logits, arrived, width, topk_w, topk_e, shared_gate,
                                      offsets, rows, dest, tokens, experts, k, renormalize, scale, n_groups, groups_keep, tile_rows,
                                      tile_expert, tile_row0, tile_info, stream);
 }
@@ -174,7 +179,8 @@ extern "C" int ix_moe_route_dispatch_small(const void* x, int dtype, const void*
 // is what is routed, and h [tokens, width] float32 becomes h + delta.  delta and x_out are of `dtype`.
 extern "C" int ix_moe_norm_route_dispatch_small(float* h, const void* delta, int dtype, const void* gamma,
                                                 int gamma_dtype, float eps, void* x_out, const void* wr, int wr_dtype,
-                                                const void* shared_gate_w, int sg_dtype, float* logits,
+                                                const void* shared_gate_w, int sg_dtype, const float* bias,
+                                                float* logits,
                                                 int32_t* arrived, int64_t width, float* topk_w, int32_t* topk_e,
                                                 float* shared_gate, int32_t* offsets, int32_t* rows, int32_t* dest,
                                                 int tokens, int experts, int k, int renormalize, float scale, int n_groups, int groups_keep,
@@ -183,7 +189,7 @@ extern "C" int ix_moe_norm_route_dispatch_small(float* h, const void* delta, int
   IX_REQUIRE(h && delta && gamma && x_out, "h, delta, gamma and x_out needed");
   IX_REQUIRE(gamma_dtype == IX_F32 || gamma_dtype == IX_BF16, "the norm weight must be float32 or bfloat16");
   return route_dispatch_small_launch(nullptr, h, delta, gamma, gamma_dtype, eps, x_out, dtype, wr, wr_dtype,
-                                     shared_gate_w, sg_dtype, logits, arrived, width, topk_w, topk_e, shared_gate,
+                                     shared_gate_w, sg_dtype, bias, logits, arrived, width, topk_w, topk_e, shared_gate,
                                      offsets, rows, dest, tokens, experts, k, renormalize, scale, n_groups, groups_keep, tile_rows,
                                      tile_expert, tile_row0, tile_info, stream);
 }

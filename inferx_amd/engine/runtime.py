@@ -129,13 +129,13 @@ class Runtime:
     def gated_linear(self, x: torch.Tensor, w_gate_up: torch.Tensor, limit: float = 0.0,
                      bias: Optional[torch.Tensor] = None) -> torch.Tensor:
         """silu(x . Wg^T) * (x . Wu^T) for w_gate_up = [Wg; Wu] of shape [2 n, in] -> [T, n].  `bias` (2 n numbers) is
-        added to both products first; with `limit` > 0 they meet in the clamped form instead (`ops.glu_bias`)."""
+        added to both products first; with `limit` other than 0 they meet in another form (see `ops.glu_bias`)."""
         from .. import ops
         if bias is None and self._skinny_ok(x, w_gate_up):
             return self._skinny(x, w_gate_up, True, limit)
         gate_up = self.linear(x, w_gate_up)
         act = self.empty((x.shape[0], w_gate_up.shape[0] // 2))
-        if bias is None and limit <= 0:
+        if bias is None and limit == 0:
             ops.silu_mul(gate_up, act)
         else:
             ops.glu_bias(gate_up, bias, act, limit)

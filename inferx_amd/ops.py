@@ -232,12 +232,19 @@ def _check_caches(q, k_cache, v_cache):
           "value cache must be [pages, kv_heads, d, page_size]")
 
 
+def key_span(window: int, chunk: int) -> int:
+    """How far back attention's queries read, as the one number that its kernels take: 0 every earlier position, W > 0
+    the last W (the query's own included), -C < 0 those of the query's own chunk of C positions."""
+    _need(window >= 0 and chunk >= 0 and not (window and chunk), "a window or chunks, neither negative")
+    return window or -chunk
+
+
 def attention_plain(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, block_table: torch.Tensor,
                     seq_of_token: torch.Tensor, positions: torch.Tensor, out: torch.Tensor, scale: float,
-                    window: int, sink: Optional[torch.Tensor] = None, turn_back: Optional[torch.Tensor] = None,
+                    span: int, sink: Optional[torch.Tensor] = None, turn_back: Optional[torch.Tensor] = None,
                     softcap: float = 0.0) -> None:
     """Paged attention, one workgroup per (token, head).  q [T, heads, d], out [T, heads, value size] (the value
-    cache's).  `sink` float32 [heads]: exp(sink) joins every softmax's denominator, with no key and no value.
+    cache's).  `span`: how far back a query reads, see `key_span`.  `sink` float32 [heads]: exp(sink) joins every softmax's denominator, with no key and no value.
     `turn_back` float32 [T, value size / 2, 2]: every head's result is rotated by minus these angles (halves paired).
     `softcap` c > 0: scores become c tanh(score / c)."""
     T, heads, d = q.shape
@@ -254,7 +261,7 @@ def attention_plain(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tenso
     _is_i32(positions, T)
     _call("ix_attention_plain", _ptr(q), _ptr(k_cache), _ptr(v_cache), _i32(_dt(q)), _ptr(block_table),
           _ptr(seq_of_token), _ptr(positions), _ptr(out), _i64(T), _i32(heads), _i32(kv_heads), _i32(d), _i32(vd),
-          _i32(page_size), _i32(block_table.shape[1]), _f32(scale), _i32(window), _ptr(sink), _ptr(turn_back), _f32(softcap), _stream())
+          _i32(page_size), _i32(block_table.shape[1]), _f32(scale), _i32(span), _ptr(sink), _ptr(turn_back), _f32(softcap), _stream())
 
 
 def qkv_norm_rope_append(qkv: torch.Tensor, q_norm: Optional[torch.Tensor], k_norm: Optional[torch.Tensor], eps: float,
@@ -310,7 +317,7 @@ def rotate_heads(x: torch.Tensor, cos_sin: torch.Tensor, inverse: bool = False) 
 
 def attention_mfma(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, block_table: torch.Tensor,
                    tiles: torch.Tensor, positions: torch.Tensor, out: torch.Tensor, n_splits: int,
-                   workspace: Optional[torch.Tensor], scale: float, window: int, tile_queries: int = 16,
+                   workspace: Optional[torch.Tensor], scale: float, span: int, tile_queries: int = 16,
                    prefetch: bool = False, grouped: bool = False, sink: Optional[torch.Tensor] = None,
                    turn_back: Optional[torch.Tensor] = None, softcap: float = 0.0,
                    gate: Optional[torch.Tensor] = None) -> None:
@@ -341,7 +348,7 @@ def attention_mfma(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor
     args = (_ptr(q), _ptr(k_cache), _ptr(v_cache), _ptr(block_table), _ptr(tiles[0]),
             _ptr(tiles[1]), _ptr(tiles[2]), _ptr(positions), _ptr(out), _ptr(part_o), _ptr(part_ml), _i64(T),
             _i32(n_tiles), _i32(tile_queries), _i32(n_splits), _i32(heads), _i32(kv_heads), _i32(d), _i32(page_size),
-            _i32(block_table.shape[1]), _f32(scale), _i32(window), _i32(1 if prefetch else 0),
+            _i32(block_table.shape[1]), _f32(scale), _i32(span), _i32(1 if prefetch else 0),
             _i32(1 if grouped else 0))
     if sink is None and turn_back is None and softcap <= 0 and gate is None:
         _call("ix_attention_mfma", *args, _stream())
@@ -367,7 +374,7 @@ def _gate_rows(gate: Optional[torch.Tensor], tokens: int, width: int, dtype):
 
 
 def attention_prefill(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, block_table: torch.Tensor,
-                      tiles: torch.Tensor, positions: torch.Tensor, out: torch.Tensor, scale: float, window: int,
+                      tiles: torch.Tensor, positions: torch.Tensor, out: torch.Tensor, scale: float, span: int,
                       tile_queries: int = 64, pairs: Optional[torch.Tensor] = None, n_splits: int = 1,
                       workspace: Optional[torch.Tensor] = None, sink: Optional[torch.Tensor] = None,
                       softcap: float = 0.0, gate: Optional[torch.Tensor] = None) -> None:
@@ -414,7 +421,7 @@ def attention_prefill(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Ten
         _call("ix_attention_prefill128", _ptr(q), _ptr(k_cache), _ptr(v_cache), _ptr(block_table), _ptr(tiles[0]),
               _ptr(tiles[1]), _ptr(tiles[2]), _ptr(pairs[0]), _ptr(pairs[1]), _i32(pairs.shape[1]), _ptr(positions),
               _ptr(out), _ptr(part_o), _ptr(part_ml), _i32(n_splits), _i64(T), _i32(tiles.shape[1]), _i32(heads),
-              _i32(kv_heads), _i32(d), _i32(page_size), _i32(block_table.shape[1]), _f32(scale), _i32(window),
+              _i32(kv_heads), _i32(d), _i32(page_size), _i32(block_table.shape[1]), _f32(scale), _i32(span),
               _ptr(sink), _f32(softcap), gate_ptr, _i64(gate_stride), _stream())
         return
     _need(sink is None and softcap <= 0 and gate is None, "sinks, capped scores and gates take tiles of 128 queries")
@@ -422,7 +429,7 @@ def attention_prefill(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Ten
           _ptr(tiles[1]), _ptr(tiles[2]), _ptr(pairs[0]), _ptr(pairs[1]), _i32(pairs.shape[1]), _ptr(positions),
           _ptr(out), _ptr(part_o), _ptr(part_ml), _i32(n_splits), _i64(T), _i32(tiles.shape[1]), _i32(tile_queries),
           _i32(heads), _i32(kv_heads), _i32(d), _i32(page_size), _i32(block_table.shape[1]), _f32(scale),
-          _i32(window), _stream())
+          _i32(span), _stream())
 
 
 ROUTE_SMALL_TOKENS = 128
@@ -436,14 +443,15 @@ def route_mode(renormalize: bool, sigmoid: bool = False, group_top2: bool = Fals
 def moe_route(x: torch.Tensor, router_w: torch.Tensor, shared_gate_w: Optional[torch.Tensor], topk_w: torch.Tensor,
               topk_e: torch.Tensor, shared_gate: Optional[torch.Tensor], renormalize: bool, scale: float,
               always: int = 0, groups: int = 1, groups_keep: int = 1, sigmoid: bool = False,
-              group_top2: bool = False) -> None:
+              group_top2: bool = False, bias: Optional[torch.Tensor] = None) -> None:
     """Router product, softmax and top-k in float32; optional sigmoid gate of the shared expert.
     `sigmoid`: an expert's score is sigmoid(z) of its own logit instead of the softmax over all; `group_top2`: a
     group's score is the sum of its two largest scores instead of its largest.
     `always`: that many further slots per token after the chosen ones (topk_w and topk_e are [T, k + always]), naming
     the experts E .. E + always - 1 with the shared gate's value (or 1) as their weight: experts that every token uses.
     `groups`, `groups_keep`: the experts form that many equal groups of neighbours, and only experts of the
-    `groups_keep` groups with the largest best score can be chosen (1, 1: every expert can)."""
+    `groups_keep` groups with the largest best score can be chosen (1, 1: every expert can).
+    `bias` float32 [experts]: added to the product before anything else."""
     T, H = x.shape
     E = router_w.shape[0]
     k = topk_w.shape[1] - always
@@ -457,6 +465,7 @@ def moe_route(x: torch.Tensor, router_w: torch.Tensor, shared_gate_w: Optional[t
         _need(shared_gate_w.numel() == H, "shared gate weight must hold `hidden` numbers")
         _need(shared_gate is not None and shared_gate.dtype == torch.float32 and shared_gate.numel() >= T,
               "shared_gate must be float32 [T]")
+    _router_bias(bias, E)
     scratch = None
     all_bf16 = (x.dtype == torch.bfloat16 and router_w.dtype == torch.bfloat16
                 and (shared_gate_w is None or shared_gate_w.dtype == torch.bfloat16))
@@ -465,10 +474,14 @@ def moe_route(x: torch.Tensor, router_w: torch.Tensor, shared_gate_w: Optional[t
         # bfloat16: the scores are a product on the matrix cores
         scratch = torch.empty((T, E + 1), dtype=torch.float32, device=x.device)
     _call("ix_moe_route", _ptr(x), _i32(_dt(x)), _ptr(router_w), _i32(_dt(router_w)), _ptr(shared_gate_w),
-          _i32(_dt(shared_gate_w) if shared_gate_w is not None else F32), _ptr(topk_w), _ptr(topk_e),
+          _i32(_dt(shared_gate_w) if shared_gate_w is not None else F32), _ptr(bias), _ptr(topk_w), _ptr(topk_e),
           _ptr(shared_gate if shared_gate_w is not None else None), _ptr(scratch), _i64(T), _i64(H), _i32(E), _i32(k),
           _i32(route_mode(renormalize, sigmoid, group_top2)), _f32(scale), _i32(always), _i32(groups),
           _i32(groups_keep), _stream())
+
+
+def _router_bias(bias: Optional[torch.Tensor], experts: int) -> None:
+    _need(bias is None or (bias.dtype == torch.float32 and bias.numel() == experts), "the router's bias must be float32 [experts]")
 
 
 # the one-launch router: at most this many tokens, experts and bytes of one token as float32
@@ -499,7 +512,7 @@ def moe_route_dispatch(x: Optional[torch.Tensor], router_w: torch.Tensor, shared
                        renormalize: bool, scale: float, offsets: torch.Tensor, rows: torch.Tensor,
                        dest: torch.Tensor, tile_rows: int = 0, tile_map: Optional[torch.Tensor] = None,
                        norm: Optional[tuple] = None, groups: int = 1, groups_keep: int = 1, sigmoid: bool = False,
-                       group_top2: bool = False) -> None:
+                       group_top2: bool = False, bias: Optional[torch.Tensor] = None) -> None:
     """`moe_route` and `moe_dispatch` for up to 16 tokens in one launch: the router scores are spread over many
     workgroups, and the last one to finish its scores selects and groups (`route_one_launch_fits`).
 
@@ -536,9 +549,10 @@ def moe_route_dispatch(x: Optional[torch.Tensor], router_w: torch.Tensor, shared
         _need(tile_map is not None, "tile_map needed")
         _is_i32(tile_map, 2 * mt + 1)
         te, tr, ti = tile_map[:mt], tile_map[mt:2 * mt], tile_map[2 * mt:]
+    _router_bias(bias, E)
     logits = torch.empty((T, E + 1), dtype=torch.float32, device=x.device)
     router = (_ptr(router_w), _i32(_dt(router_w)), _ptr(shared_gate_w),
-              _i32(_dt(shared_gate_w) if shared_gate_w is not None else F32), _ptr(logits),
+              _i32(_dt(shared_gate_w) if shared_gate_w is not None else F32), _ptr(bias), _ptr(logits),
               _ptr(_arrival_counter(x.device)), _i64(H), _ptr(topk_w), _ptr(topk_e),
               _ptr(shared_gate if shared_gate_w is not None else None), _ptr(offsets), _ptr(rows), _ptr(dest),
               _i32(T), _i32(E), _i32(k), _i32(route_mode(renormalize, sigmoid, group_top2)), _f32(scale), _i32(groups),
@@ -573,6 +587,9 @@ def moe_dispatch(topk_e: torch.Tensor, offsets: torch.Tensor, rows: torch.Tensor
 
 
 PLAIN_PRODUCT, GATE_UP_SWIGLU, RELU_SQUARED = 0, 1, 2
+# what a gated product does with gate and up, as one number (the kernels' `limit`): 0 silu(g) * u, a limit > 0 the clamped
+# form, this one gelu(g) * u in gelu's tanh form
+GLU_GELU_TANH = -1.0
 
 
 def _epilogue(gate_up) -> int:
@@ -1307,10 +1324,11 @@ def attention_diff_mfma(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.T
           _i32(1 if grouped else 0), _stream())
 
 
-# ---- a gated product's activation with biases and limits; two branches added to the stream ---------------------
+# ---- a gated product's activation with biases and limits; branches added to the stream -----------------------------
 def glu_bias(gate_up: torch.Tensor, bias: Optional[torch.Tensor], out: torch.Tensor, limit: float = 0.0) -> None:
     """out[t, i] = glu(gate_up[t, i] + bias[i], gate_up[t, W + i] + bias[W + i]); glu(g, u) = silu(g) * u, or with
-    `limit` > 0 the clamped form g' sigmoid(1.702 g') (u' + 1), g' = min(g, limit), u' = clamp(u, -limit, limit)."""
+    `limit` > 0 the clamped form g' sigmoid(1.702 g') (u' + 1), g' = min(g, limit), u' = clamp(u, -limit, limit), or with
+    `GLU_GELU_TANH` gelu(g) * u."""
     T, W2 = gate_up.shape
     _need(W2 % 2 == 0 and out.shape == (T, W2 // 2) and out.dtype == gate_up.dtype, "shape or dtype mismatch")
     _need(bias is None or bias.numel() == W2, "the bias holds the gate's numbers, then the up's")
@@ -1318,14 +1336,59 @@ def glu_bias(gate_up: torch.Tensor, bias: Optional[torch.Tensor], out: torch.Ten
           _i32(_dt(out)), _i64(T), _i64(W2 // 2), _f32(limit), _stream())
 
 
-def add_branches(h: torch.Tensor, a: torch.Tensor, b: Optional[torch.Tensor] = None,
-                 bias: Optional[torch.Tensor] = None) -> None:
-    """h [T, W] float32 += a + b + bias (b and bias optional), summed in float32."""
-    _need(h.dtype == torch.float32 and h.dim() == 2, "the residual stream is float32 [T, W]")
-    _need(a.shape == h.shape and (b is None or (b.shape == h.shape and b.dtype == a.dtype)), "the branches have h's shape")
-    _need(bias is None or bias.numel() == h.shape[1], "one bias per column")
-    _call("ix_add_branches", _ptr(h), _ptr(a), _ptr(b), _i32(_dt(a)), _ptr(bias),
-          _i32(_dt(bias) if bias is not None else F32), _i64(h.shape[0]), _i64(h.shape[1]), _stream())
+def branch_norm(h: torch.Tensor, a: Optional[torch.Tensor] = None, b: Optional[torch.Tensor] = None,
+                bias: Optional[torch.Tensor] = None, experts: Optional[tuple] = None,
+                again: Optional[tuple] = None, step: Optional[torch.Tensor] = None, norms=(), eps: float = 0.0,
+                rows: Optional[torch.Tensor] = None) -> None:
+    """h [T, W] float32 += (a + b + bias + experts' sum) + again + step, every term optional, and up to two RMS norms of
+    the result in the same pass (`norms`: (weight, out) each, out of the activations' type).
+    `experts` = (y, dest, topk_w, shared or None, shared_gate or None) as for `moe_combine`; `again` = (table, ids, scale):
+    table[ids[t]] * scale, or table[t] * scale without ids; `bias`, `step`: W numbers.  With `rows` (int32) only those
+    rows are normalised and h stays as it is."""
+    T, W = h.shape
+    _need(h.dtype == torch.float32, "the residual stream is float32 [T, W]")
+    dense = [t for t in (a, b) if t is not None]
+    y = dest = topk_w = shared = gate = None
+    k = 0
+    if experts is not None:
+        y, dest, topk_w, shared, gate = experts
+        k = topk_w.shape[1]
+        _need(topk_w.shape[0] == T and topk_w.dtype == torch.float32 and y.shape[1] == W and y.shape[0] >= T * k,
+              "the experts' rows do not fit")
+        _is_i32(dest, T * k)
+        _need(gate is None or (gate.dtype == torch.float32 and gate.numel() >= T), "the shared gate must be float32 [T]")
+        dense += [] if shared is None else [shared]
+    for t in dense:
+        _need(t.shape == h.shape, "a branch's result must have the shape of h")
+    outs = [o for _, o in norms]
+    types = {t.dtype for t in dense + outs + ([y] if y is not None else [])}
+    _need(len(types) <= 1, "the branches and the normalised rows must be of one type")
+    dtype = _dt(next(t for t in dense + outs + ([y] if y is not None else []))) if types else F32
+    _need(len(norms) <= 2, "at most two norms")
+    n = T
+    if rows is not None:
+        _need(len(norms) > 0, "picked rows are for a norm's result")
+        n = outs[0].shape[0]
+        _is_i32(rows, n)
+    for w, o in norms:
+        _need(w.numel() == W and o.shape == (n, W), "a norm's weight or result does not fit")
+    for v in (bias, step):
+        _need(v is None or v.numel() == W, "one number per column")
+    table = ids = None
+    scale, table_rows = 1.0, 0
+    if again is not None:
+        table, ids, scale = again
+        _need(table.dim() == 2 and table.shape[1] == W, "the table's width differs from h")
+        table_rows = table.shape[0]
+        _need(ids is not None or table_rows >= T, "a row per token, or ids")
+        if ids is not None:
+            _is_i32(ids, T)
+    code = lambda t: _i32(_dt(t) if t is not None else F32)
+    (w1, o1), (w2, o2) = (list(norms) + [(None, None), (None, None)])[:2]
+    _call("ix_branch_norm", _ptr(h), _i32(dtype), _ptr(a), _ptr(b), _ptr(bias), code(bias), _ptr(y), _ptr(dest), _ptr(topk_w),
+          _i32(k), _ptr(shared), _ptr(gate if shared is not None else None), _ptr(table), code(table), _ptr(ids),
+          _i64(table_rows), _f32(scale), _ptr(step), code(step), _ptr(w1), code(w1), _ptr(o1), _ptr(w2), code(w2), _ptr(o2),
+          _ptr(rows), _i64(n), _i64(W), _f32(eps), _stream())
 
 
 # ---- recurrent mixers with a matrix of state per head ---------------------------------------------------------------
@@ -1504,6 +1567,15 @@ def latent_prepare(q: torch.Tensor, dkv: torch.Tensor, norm_w: torch.Tensor, eps
           _i32(q_dim), _i32(rot_dim), _i32(rank), _i32(1 if halves else 0), _stream())
 
 
+def _head_gate(gate: Optional[torch.Tensor], tokens: int, heads: int, dtype):
+    """(address, row stride) of a gate with a number per token and head."""
+    if gate is None:
+        return None, 0
+    _need(gate.shape == (tokens, heads) and gate.stride(1) == 1 and gate.dtype == dtype and gate.is_cuda,
+          "the gate must be rows of one number per head")
+    return gate.data_ptr(), gate.stride(0)
+
+
 def _head_rows(t: torch.Tensor, tokens: int, heads: int, n: int, what: str):
     """(token stride, head stride) of a tensor indexed [token, head, i] whose last dimension is dense."""
     _need(t.dim() == 3 and t.shape[0] == tokens and t.shape[1] == heads and t.shape[2] >= n and t.stride(2) == 1
@@ -1513,10 +1585,11 @@ def _head_rows(t: torch.Tensor, tokens: int, heads: int, n: int, what: str):
 
 def latent_attention_plain(q_lat: torch.Tensor, q_rot: torch.Tensor, cache: torch.Tensor, block_table: torch.Tensor,
                            seq_of_token: torch.Tensor, positions: torch.Tensor, out: torch.Tensor, rank: int,
-                           rot_dim: int, scale: float, window: int = 0) -> None:
+                           rot_dim: int, scale: float, window: int = 0, head_gate: Optional[torch.Tensor] = None) -> None:
     """Causal attention of queries [token, head] over cached rows [c | kr]: score = (q_lat . c + q_rot . kr) * scale,
     softmax in float32, out = sum of weights * c.  `window` W > 0: a query reads its own and the W - 1 rows before.  q_lat, out [token, head, rank] and q_rot [token, head, rot_dim] are
-    views with any token and head strides; cache [pages, 1, page_size, rank + rot_dim]."""
+    views with any token and head strides; cache [pages, 1, page_size, rank + rot_dim].  `head_gate` [token, head] (rows
+    may be strided): every head's result is multiplied by the sigmoid of its number."""
     T, heads = q_lat.shape[0], q_lat.shape[1]
     ql_t, ql_h = _head_rows(q_lat, T, heads, rank, "q_lat")
     qr_t, qr_h = _head_rows(q_rot, T, heads, rot_dim, "q_rot")
@@ -1531,7 +1604,7 @@ def latent_attention_plain(q_lat: torch.Tensor, q_rot: torch.Tensor, cache: torc
     _call("ix_latent_attention_plain", q_lat.data_ptr(), _i64(ql_t), _i64(ql_h), q_rot.data_ptr(), _i64(qr_t), _i64(qr_h),
           _ptr(cache), _i32(_dt(q_lat)), _ptr(block_table), _ptr(seq_of_token), _ptr(positions), out.data_ptr(),
           _i64(o_t), _i64(o_h), _i64(T), _i32(heads), _i32(rank), _i32(rot_dim), _i32(cache.shape[2]),
-          _i32(block_table.shape[1]), _f32(scale), _i32(window), _stream())
+          _i32(block_table.shape[1]), _f32(scale), _i32(window), *_head_gate(head_gate, T, heads, q_lat.dtype), _stream())
 
 
 LATENT_MFMA_MAX_SPLITS = 32
@@ -1560,7 +1633,8 @@ def latent_mfma_splits(tokens: int, heads: int) -> int:
 def latent_attention_mfma(q_lat: torch.Tensor, q_rot: torch.Tensor, cache: torch.Tensor, block_table: torch.Tensor,
                           seq_of_token: torch.Tensor, positions: torch.Tensor, out: torch.Tensor, rank: int,
                           rot_dim: int, scale: float, one_token_each: bool = False, n_splits: int = 1,
-                          work: Optional[Tuple[torch.Tensor, torch.Tensor]] = None, window: int = 0) -> None:
+                          work: Optional[Tuple[torch.Tensor, torch.Tensor]] = None, window: int = 0,
+                          head_gate: Optional[torch.Tensor] = None) -> None:
     """`latent_attention_plain` on the matrix cores (see `latent_mfma_fits`).  `one_token_each`: every request brings
     one token; its keys may then be cut into `n_splits` slices, with `work` = float32 ([T * heads * n_splits, rank],
     [T * heads * n_splits, 2]) and a contiguous `out` [T, heads, rank]."""
@@ -1587,4 +1661,4 @@ def latent_attention_mfma(q_lat: torch.Tensor, q_rot: torch.Tensor, cache: torch
           _ptr(cache), _ptr(block_table), _ptr(seq_of_token), _ptr(positions), out.data_ptr(), _i64(o_t), _i64(o_h),
           _ptr(part_o), _ptr(part_ml), _i32(n_splits), _i64(T), _i32(heads), _i32(rank), _i32(rot_dim),
           _i32(cache.shape[2]), _i32(block_table.shape[1]), _f32(scale), _i32(1 if one_token_each else 0), _i32(window),
-          _stream())
+          *_head_gate(head_gate, T, heads, q_lat.dtype), _stream())

@@ -14,6 +14,14 @@ keys) and `value_position` (a position encoding over ALL of a value head: the va
 by j, and every head's weighted sum at position i is rotated back by i, so that what a query receives depends on
 i - j only).  With any of these the step after the product is `ops.qkv_norm_rope_append`; with values of another size
 the attention itself is the plain kernel.  `softcap` c > 0: a score becomes c tanh(score / c) before the softmax.
+`chunk` C > 0 (instead of a window): the sequence falls into chunks of C positions, counted from its start, and a query
+reads the keys of its own chunk up to its own position; the pages of passed chunks are given back.
+
+`pad`: a bfloat16 run arranges the heads for the matrix-core kernels when the weights are bound.  Those take values as wide
+as keys and the fused steps rotate whole heads of a multiple of 32 numbers in pairs (i, i + half): every head gets the
+next such size, by rows of zeros in Wq, Wk and Wv and columns of zeros in Wo, and where a part of the head is rotated its
+rows are put so that the pairs are those of the whole head, the rest under pairs of frequency zero.  One order for queries
+and keys changes no score.
 """
 from __future__ import annotations
 
@@ -35,15 +43,16 @@ class PagedAttention(Mixer):
                  out_bias: bool = False, window: int = 0, scale: Optional[float] = None,
                  position: Optional[PartSpec] = None, init_std: float = 0.02, value_dim: Optional[int] = None,
                  qk_norm: bool = False, qk_norm_eps: float = 1e-6, sink: bool = False,
-                 value_position: Optional[PartSpec] = None, softcap: float = 0.0):
+                 value_position: Optional[PartSpec] = None, softcap: float = 0.0, chunk: int = 0, pad: bool = False):
         if num_heads % num_kv_heads:
             raise ValueError(f"num_heads {num_heads} is not a multiple of num_kv_heads {num_kv_heads}")
-        general = qk_norm or value_position is not None or (value_dim is not None and int(value_dim) != int(head_dim))
+        general = qk_norm or value_position is not None or (value_dim is not None and int(value_dim) != int(head_dim)) or pad
         if head_dim > 256 or (head_dim % 2 and not general):  # (the step after the product for plain heads pairs elements)
             raise ValueError(f"head_dim {head_dim} must be even and at most 256")
         self.out_bias = bool(out_bias)
         self.hidden_size, self.num_heads, self.num_kv_heads = int(hidden_size), int(num_heads), int(num_kv_heads)
-        self.head_dim, self.qkv_bias, self.window = int(head_dim), bool(qkv_bias), int(window)
+        self.head_dim, self.qkv_bias, self.window, self.chunk = int(head_dim), bool(qkv_bias), int(window), int(chunk)
+        self.span = ops.key_span(self.window, self.chunk)  # how far back a query reads, as the kernels take it
         self.scale = float(scale) if scale is not None else self.head_dim ** -0.5
         self.init_std, self.softcap = float(init_std), float(softcap)
         if self.softcap < 0:
@@ -58,6 +67,7 @@ class PagedAttention(Mixer):
                 raise ValueError(f"the position encoding rotates elements {begin} to {begin + dim} of heads of "
                                  f"{self.head_dim}: an even number of elements within the head is needed")
         self.value_dim = self.head_dim if value_dim is None else int(value_dim)
+        self.pad, self.key_size, self.value_size = bool(pad), self.head_dim, self.value_dim  # (sizes in the checkpoint)
         self.qk_norm, self.qk_norm_eps, self.has_sink = bool(qk_norm), float(qk_norm_eps), bool(sink)
         self.value_position = build_part("position", value_position) if value_position is not None else None
         if self.value_dim <= 0 or self.value_dim > 256:
@@ -66,10 +76,15 @@ class PagedAttention(Mixer):
                                                 getattr(self.value_position, "rotary_dim", 0) != self.value_dim):
             raise ValueError("the values' position encoding must rotate all of a value head")
         # the step after the product that knows norms per head, rotated values and values of another size
-        self.general = self.qk_norm or self.value_position is not None or self.value_dim != self.head_dim
+        self.general = self._needs_general_step()
+        if self.pad and (self.qk_norm or self.value_position is not None):
+            raise ValueError("heads with norms of their own or rotated values are not arranged anew")
         if self.general and self.qkv_bias:
             raise ValueError("biases on q, k, v do not go with norms per head, rotated values or values of another size")
         self.w_qkv = self.b_qkv = self.w_out = self.b_out = self.q_norm = self.k_norm = self.sink = None
+
+    def _needs_general_step(self) -> bool:
+        return self.qk_norm or self.value_position is not None or self.value_dim != self.head_dim or self.head_dim % 2 != 0
 
     @property
     def q_dim(self) -> int:
@@ -89,7 +104,7 @@ class PagedAttention(Mixer):
 
     def cache_need(self) -> CacheNeed:
         return CacheNeed.keys_and_values(self.num_kv_heads, self.head_dim, self.window,
-                                         None if self.value_dim == self.head_dim else self.value_dim)
+                                         None if self.value_dim == self.head_dim else self.value_dim, self.chunk)
 
     def subparts(self):
         return [self.position, self.value_position]
@@ -110,7 +125,43 @@ class PagedAttention(Mixer):
             specs.append(ParamSpec("o_proj.bias", (H,), std=s))
         return specs
 
+    def _arrange_heads(self, tensors):
+        """The heads as `pad` describes; returns the tensors with their rows (and Wo's columns) in place."""
+        H, G, d, vd = self.num_heads, self.num_kv_heads, self.key_size, self.value_size
+        D = padded_head(d, vd, to=32)
+        begin, dims = self.rotated if self.position is not None else (0, 0)
+        places = list(range(begin, begin + dims // 2)) + [-1] * (D // 2 - dims // 2)           # which row goes to place i ..
+        places += list(range(begin + dims // 2, begin + dims)) + [-1] * (D // 2 - dims // 2)   # .. and to i + D / 2
+        rest = [j for j in range(d) if not begin <= j < begin + dims]
+        for i, p in enumerate(places):
+            if p < 0 and rest:
+                places[i] = rest.pop(0)
+        if self.position is None or (D == d and (begin, dims) == (0, D)):
+            places = list(range(d)) + [-1] * (D - d)
+
+        def put(t, heads):
+            t = t.unflatten(0, (heads, d))
+            out = t.new_zeros((heads, D) + tuple(t.shape[2:]))
+            here = [i for i, p in enumerate(places) if p >= 0]
+            out[:, here] = t[:, [places[i] for i in here]]
+            return out.flatten(0, 1)
+
+        out = dict(tensors)
+        for kind in ("weight", "bias"):
+            if f"q_proj.{kind}" in tensors:
+                out[f"q_proj.{kind}"], out[f"k_proj.{kind}"] = put(tensors[f"q_proj.{kind}"], H), put(tensors[f"k_proj.{kind}"], G)
+                out[f"v_proj.{kind}"] = pad_heads(tensors[f"v_proj.{kind}"], G, vd, D)
+        out["o_proj.weight"] = pad_heads(tensors["o_proj.weight"], H, vd, D, dim=1)
+        self.head_dim = self.value_dim = D
+        if self.position is not None:
+            self.rotated = (0, D)
+            self.position.widen(D // 2)
+        self.general = self._needs_general_step()
+        return out
+
     def bind(self, tensors, rt) -> None:
+        if self.pad and rt.dtype == torch.bfloat16:
+            tensors = self._arrange_heads(tensors)
         self.w_qkv = stack_rows([tensors[f"{n}_proj.weight"] for n in "qkv"])
         self.b_qkv = stack_rows([tensors[f"{n}_proj.bias"] for n in "qkv"]) if self.qkv_bias else None
         self.w_out = tensors["o_proj.weight"].contiguous()
@@ -181,7 +232,7 @@ class PagedAttention(Mixer):
                 tile = WIDE_PREFILL_TILE if self.head_dim % 32 == 0 else PREFILL_TILE
                 lds_fits = (self.head_dim <= 128 and page_size & (page_size - 1) == 0
                             and (not special or (turn_back is None and tile == WIDE_PREFILL_TILE)))
-                lds, waves = mixed_step_plan(ctx, self.window, self.num_heads, self.num_kv_heads, lds_fits, tile)
+                lds, waves = mixed_step_plan(ctx, self.span, self.num_heads, self.num_kv_heads, lds_fits, tile)
                 table = ctx.block_tables[cache.group]
                 if lds is not None:
                     tiles, pairs, slices = lds
@@ -190,7 +241,7 @@ class PagedAttention(Mixer):
                         work = ctx.rt.empty((T * self.num_heads * slices * (self.head_dim + 2),), torch.float32)
                     shared = {"sink": self.sink, "softcap": self.softcap, "gate": gate} if special else {}
                     ops.attention_prefill(q, cache.k, cache.v, table, tiles, ctx.positions, out, self.scale,
-                                          self.window, tile, pairs, slices, work, **shared)
+                                          self.span, tile, pairs, slices, work, **shared)
                 for rows, tiles, positions, n_splits, grouped in waves:
                     # a launch that serves some of the step's requests gets their rows put side by side
                     qs = q if rows is None else q.index_select(0, rows)
@@ -204,22 +255,37 @@ class PagedAttention(Mixer):
                         work = ctx.rt.empty((qs.shape[0] * self.num_heads * n_splits * (self.head_dim + 2),),
                                             torch.float32)
                     ops.attention_mfma(qs, cache.k, cache.v, table, tiles, positions, outs, n_splits, work,
-                                       self.scale, self.window, QUERY_TILE, grouped=grouped, **more)
+                                       self.scale, self.span, QUERY_TILE, grouped=grouped, **more)
                     if rows is not None:
                         out.index_copy_(0, rows, outs)
                 return
-            tiles, tile, n_splits, grouped = query_tiles(ctx, self.window, self.num_heads, self.head_dim,
+            tiles, tile, n_splits, grouped = query_tiles(ctx, self.span, self.num_heads, self.head_dim,
                                                          self.num_kv_heads)
             work = None
             if n_splits > 1:
                 work = ctx.rt.empty((q.shape[0] * self.num_heads * n_splits * (self.head_dim + 2),), torch.float32)
             ops.attention_mfma(q, cache.k, cache.v, ctx.block_tables[cache.group], tiles, ctx.positions, out,
-                               n_splits, work, self.scale, self.window, tile, prefetch=True, grouped=grouped, **more)
+                               n_splits, work, self.scale, self.span, tile, prefetch=True, grouped=grouped, **more)
         else:
             ops.attention_plain(q, cache.k, cache.v, ctx.block_tables[cache.group], ctx.seq_of_token, ctx.positions,
-                                out, self.scale, self.window, self.sink, turn_back, self.softcap)
+                                out, self.scale, self.span, self.sink, turn_back, self.softcap)
             if gate is not None:
                 ops.sigmoid_gate(out.view(out.shape[0], -1), gate)
+
+
+def padded_head(*sizes: int, to: int = 16) -> int:
+    """The next multiple of `to` that holds all of these head sizes."""
+    return -(-max(sizes) // to) * to
+
+
+def pad_heads(t: torch.Tensor, heads: int, size: int, to: int, dim: int = 0) -> torch.Tensor:
+    """`t` has heads * size entries along `dim`; every head gets zeros after its own up to `to`."""
+    if size == to:
+        return t
+    shape = list(t.shape)
+    out = torch.zeros(shape[:dim] + [heads, to] + shape[dim + 1:], dtype=t.dtype, device=t.device)
+    out.narrow(dim + 1, 0, size).copy_(t.unflatten(dim, (heads, size)))
+    return out.flatten(dim, dim + 1)
 
 
 # ---- the wavefront-level kernel (ops.attention_mfma)
@@ -271,7 +337,7 @@ def _tiles_of(n: np.ndarray, first_row: np.ndarray, seqs: np.ndarray, tile: int)
     return np.stack([seqs[which], first_row[which] + off, rows]).astype(np.int32)
 
 
-def _pairs_by_work(t: np.ndarray, b, window: int, pair: bool, slices: int = 1) -> np.ndarray:
+def _pairs_by_work(t: np.ndarray, b, span: int, pair: bool, slices: int = 1) -> np.ndarray:
     """Which two tiles each workgroup of the LDS-sharing kernel takes, int32 [2, n_pairs].  A tile's work grows
     with the keys it reads (all up to its last query, or a window of them), so the tile that reads most is paired
     with the one that reads least, and so on inwards: workgroups then take about equally long.  Pairs are ordered
@@ -282,7 +348,8 @@ def _pairs_by_work(t: np.ndarray, b, window: int, pair: bool, slices: int = 1) -
     new = (b.q_start[1:] - b.q_start[:-1]).astype(np.int64)
     first_row = t[1] - b.q_start[:-1].astype(np.int64)[t[0]]           # the tile's first query within its portion
     end = b.seq_lens.astype(np.int64)[t[0]] - new[t[0]] + first_row + t[2]  # one past the last key it reads
-    start = np.maximum(0, end - t[2] + 1 - window) if window > 0 else np.zeros_like(end)
+    first = end - t[2]  # the position of the tile's first query
+    start = np.maximum(0, first + 1 - span) if span > 0 else (first - first % -span if span < 0 else np.zeros_like(end))
     work = -(-(end - (start // 64) * 64) // 64)  # rounds of 64 keys
     order = np.argsort(-work, kind="stable")
     half = (n_tiles + 1) // 2
@@ -306,7 +373,7 @@ def serves_group_together(heads: int, kv_heads: int) -> bool:
     return 2 <= heads // kv_heads <= 16
 
 
-def mixed_step_plan(ctx, window: int, heads: int, kv_heads: int, lds_fits: bool = True, tile: int = PREFILL_TILE):
+def mixed_step_plan(ctx, span: int, heads: int, kv_heads: int, lds_fits: bool = True, tile: int = PREFILL_TILE):
     """Who serves which requests of a step in which some request brings more than one token: (lds, waves).
 
     lds = (tiles, pairs, slices) for the LDS-sharing kernel, rows as in the step, or None.  It takes the requests
@@ -323,7 +390,8 @@ def mixed_step_plan(ctx, window: int, heads: int, kv_heads: int, lds_fits: bool 
     Sent through the LDS-sharing kernel, a decoding request would walk its whole context alone, with one query of
     a tile's 64 at work and once per query head (measured at 32 decoding requests with 4,096 keys beside two
     portions of 512, 28 query heads on 4: 487 us per layer; 162 + 57 us in two launches)."""
-    key = ("attention_mixed", window, heads, kv_heads, lds_fits, tile)
+    reach = abs(span)  # keys that a query reads at most, or 0 for all
+    key = ("attention_mixed", span, heads, kv_heads, lds_fits, tile)
     if key in ctx.memo:
         return ctx.memo[key]
     b = ctx.host
@@ -350,12 +418,12 @@ def mixed_step_plan(ctx, window: int, heads: int, kv_heads: int, lds_fits: bool 
         # eight rounds of 64 keys, 32 at most (64 tokens of 16 heads on 8,192 keys: 25 us in 16 slices against 141
         # in one; 1,024 tokens of 28 heads on 30,000 keys, 224 pairs: one slice is best).
         keys = int(b.seq_lens[seqs].max())
-        rounds = -(-(min(keys, window + tile) if window > 0 else keys) // 64)
+        rounds = -(-(min(keys, reach + tile) if reach else keys) // 64)
         slices = max(1, min(cus // (t.shape[1] * heads), rounds // PREFILL_SLICE_ROUNDS, 32))
         slices = 1 << (slices.bit_length() - 1)
     elif t is not None and t.shape[1] * heads < 8 * cus:
         keys = int(b.seq_lens[seqs].max())
-        rounds = -(-(min(keys, window + PREFILL_TILE) if window > 0 else keys) // 64)
+        rounds = -(-(min(keys, reach + PREFILL_TILE) if reach else keys) // 64)
         if rounds >= PREFILL_SLICED_MIN_ROUNDS:
             # (with two to eight workgroups per compute unit a few slices still even out what the compute units
             # get: 2,048 queries of 28 heads on 30,000 keys, 896 workgroups, 1.53 against 1.73 ms in four slices)
@@ -372,7 +440,7 @@ def mixed_step_plan(ctx, window: int, heads: int, kv_heads: int, lds_fits: bool 
         # against 15.4 ms for 24 layers).
         # (tiles of 128 queries are never paired: the workgroups are started in the order of falling work, and one
         # fills a compute unit)
-        pairs = _pairs_by_work(t, b, window, pair=not wide and slices == 1 and t.shape[1] * heads >= 2 * cus,
+        pairs = _pairs_by_work(t, b, span, pair=not wide and slices == 1 and t.shape[1] * heads >= 2 * cus,
                                slices=slices)
         lds = (to_dev(t), to_dev(pairs), slices)
         served = long.copy()
@@ -394,34 +462,34 @@ def mixed_step_plan(ctx, window: int, heads: int, kv_heads: int, lds_fits: bool 
             rows = to_dev(np.concatenate([np.arange(q_start[i], q_start[i] + n[i]) for i in seqs]))
             positions = ctx.positions.index_select(0, rows)
         units = st.shape[1] * (kv_heads if grouped else heads)
-        waves.append((rows, to_dev(st), positions, _n_splits(units, int(b.seq_lens[seqs].max()), window, QUERY_TILE),
+        waves.append((rows, to_dev(st), positions, _n_splits(units, int(b.seq_lens[seqs].max()), span, QUERY_TILE),
                       grouped))
     ctx.memo[key] = (lds, waves)
     return ctx.memo[key]
 
 
-def _n_splits(units: int, longest: int, window: int, tile: int) -> int:
+def _n_splits(units: int, longest: int, span: int, tile: int) -> int:
     """Into how many slices the wavefront-level kernel cuts each tile's keys: enough for WAVES_WANTED wavefronts,
     no slice shorter than MIN_KEYS_PER_SPLIT, a power of two (few distinct values, few captured graphs)."""
-    span = min(longest, window + tile + 32) if window > 0 else longest
-    n_splits = 1 if units >= 2048 else max(1, min(WAVES_WANTED // max(1, units), -(-span // MIN_KEYS_PER_SPLIT), 64))
+    keys = min(longest, abs(span) + tile + 32) if span else longest
+    n_splits = 1 if units >= 2048 else max(1, min(WAVES_WANTED // max(1, units), -(-keys // MIN_KEYS_PER_SPLIT), 64))
     return 1 << (n_splits.bit_length() - 1)
 
 
-def query_tiles(ctx, window: int, heads: int, head_dim: int = 128, kv_heads: Optional[int] = None):
+def query_tiles(ctx, span: int, heads: int, head_dim: int = 128, kv_heads: Optional[int] = None):
     """The wavefront-level kernel's plan: tiles (see plan_tiles), the tile size (16 or 32), into how many
     slices each tile's keys are cut, and whether a tile is one token with its grouped query heads (a step in which
     every request brings one token, and query heads share key/value heads)."""
     tile = LARGE_QUERY_TILE if (ctx.num_tokens >= LARGE_TILE_TOKENS and head_dim <= 128) else QUERY_TILE
     kv_heads = kv_heads or heads
-    key = ("attention_tiles", window, heads, kv_heads, tile)
+    key = ("attention_tiles", span, heads, kv_heads, tile)
     hit = ctx.memo.get(key)
     if hit is not None:
         return hit
     tiles_dev, n_tiles, longest = plan_tiles(ctx, tile)
     grouped = tile == QUERY_TILE and ctx.one_token_each and serves_group_together(heads, kv_heads)
     units = n_tiles * (kv_heads if grouped else heads)
-    ctx.memo[key] = (tiles_dev, tile, _n_splits(units, longest, window, tile), grouped)
+    ctx.memo[key] = (tiles_dev, tile, _n_splits(units, longest, span, tile), grouped)
     return ctx.memo[key]
 
 

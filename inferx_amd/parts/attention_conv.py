@@ -23,25 +23,10 @@ from typing import List, Optional, Tuple
 import torch
 
 from .. import ops
-from .attention import PagedAttention
+from .attention import PagedAttention, pad_heads, padded_head
 from .base import ParamSpec, StateNeed, register_part
 from .dense_mlp import stack_rows
 from .short_conv import ShortConv
-
-
-def padded_head(*sizes: int) -> int:
-    """The next multiple of sixteen that holds all of these head sizes."""
-    return -(-max(sizes) // 16) * 16
-
-
-def pad_heads(t: torch.Tensor, heads: int, size: int, to: int, dim: int = 0) -> torch.Tensor:
-    """`t` has heads * size entries along `dim`; every head gets zeros after its own up to `to`."""
-    if size == to:
-        return t
-    shape = list(t.shape)
-    out = torch.zeros(shape[:dim] + [heads, to] + shape[dim + 1:], dtype=t.dtype, device=t.device)
-    out.narrow(dim + 1, 0, size).copy_(t.unflatten(dim, (heads, size)))
-    return out.flatten(dim, dim + 1)
 
 
 class ConvAttention(PagedAttention):

@@ -12,6 +12,7 @@ object, and does not know which model it is in.  Seven kinds:
   Head              forward(ctx, x) -> float32 logits [rows, vocab]
   BranchGain        apply(delta) -> the delta with a learned gain per channel, applied where it is added
   TokenShift        forward(ctx, x, cache) -> rows blended with the rows of the tokens before them
+  StreamEntry       forward(ctx, pending, again) -> pending with what is added before a layer runs
 
 and the three tensors around a sublayer of a stream that is kept in several copies (kind "streams", see streams.py).
 
@@ -63,19 +64,26 @@ class CacheNeed:
     the last W (the query's own included), so that older pages may be given back.  Parts with equal needs share a
     group of pages (one pool, one block table per request); the runner allocates each array from this description
     and knows nothing else about it.  `keep_first`: with a window, the request's first `keep_first` tokens stay
-    readable as well (their pages are never given back)."""
+    readable as well (their pages are never given back).  `chunk` C > 0, instead of a window: only the tokens of the
+    present chunk of C positions (counted from position 0) are read again."""
 
     arrays: Tuple[CacheArray, ...]
     window: int = 0
     keep_first: int = 0
+    chunk: int = 0
+
+    def __post_init__(self):
+        if self.window < 0 or self.chunk < 0 or (self.window and self.chunk):
+            raise ValueError(f"window {self.window} and chunk {self.chunk}: not negative, and not both")
 
     @staticmethod
-    def keys_and_values(kv_heads: int, head_dim: int, window: int = 0, value_dim: Optional[int] = None) -> "CacheNeed":
+    def keys_and_values(kv_heads: int, head_dim: int, window: int = 0, value_dim: Optional[int] = None,
+                        chunk: int = 0) -> "CacheNeed":
         """Attention's cache: keys [pages, kv_heads, page_size, head_dim] and values transposed within a page
         (of `value_dim` numbers where they are not as wide as the keys)."""
         return CacheNeed((CacheArray("k", kv_heads, head_dim),
                           CacheArray("v", kv_heads, head_dim if value_dim is None else value_dim, transposed=True)),
-                         window)
+                         window, chunk=chunk)
 
 
 @dataclass(frozen=True)
@@ -190,6 +198,10 @@ class Norm(Part):
         """(weight, eps) if this is a plain RMS norm that another kernel may apply, else None."""
         return None
 
+    def forward_pair(self, ctx, h, delta, other: "Norm"):
+        """The rows of h + delta normalised by this norm and by `other`: (rows, other's rows)."""
+        return self.forward(ctx, h, delta), other.forward(ctx, h)
+
     def forward(self, ctx, h, delta=None, rows=None):
         raise NotImplementedError
 
@@ -216,6 +228,31 @@ class Mixer(Part):
 class Embedding(Part):
     def forward(self, ctx):
         """The residual stream for this step's tokens: float32 [T, hidden]."""
+        raise NotImplementedError
+
+    def again(self, ctx, h):
+        """What `forward` returned, for a model that adds it to the stream once more later (called right after
+        `forward`, before anything changes h): a tensor like h, or an `EmbeddedRows` that says how to make it."""
+        return h.clone()
+
+
+@dataclass
+class EmbeddedRows:
+    """The embedding's result as rows of its table, not formed: table[ids[t]] * scale."""
+
+    table: Any
+    ids: Any
+    scale: float = 1.0
+
+
+class StreamEntry(Part):
+    """Something the residual stream passes on its way into a layer, before the layer's norms (what is added at the
+    start of every pass of a loop).  It is named by the schedule, not by the layer."""
+
+    needs_embedding = False  # True: `again` is the embedding's result (see `Embedding.again`)
+
+    def forward(self, ctx, pending, again):
+        """`pending`: what is still to be added to the stream (or None); returns what is to be added now."""
         raise NotImplementedError
 
 
@@ -269,13 +306,13 @@ class Block:
 
 _REGISTRIES: Dict[str, Dict[str, Callable[..., Any]]] = {
     "norm": {}, "position": {}, "mixer": {}, "feed_forward": {}, "block": {}, "embedding": {}, "head": {},
-    "gain": {}, "shift": {}, "streams": {},
+    "gain": {}, "shift": {}, "streams": {}, "entry": {},
 }
 
 
 def register_part(kind: str, name: str, factory: Callable[..., Any]) -> None:
     """kind: 'norm' | 'position' | 'mixer' | 'feed_forward' | 'block' | 'embedding' | 'head' | 'gain' | 'shift' |
-    'streams'.  A block is registered by its class (see `Block`), every other kind by a callable that takes the `PartSpec`'s parameters."""
+    'streams' | 'entry'.  A block is registered by its class (see `Block`), every other kind by a callable that takes the `PartSpec`'s parameters."""
     if kind not in _REGISTRIES:
         raise KeyError(f"no such kind of part: {kind!r} (known: {', '.join(_REGISTRIES)})")
     _REGISTRIES[kind][name] = factory

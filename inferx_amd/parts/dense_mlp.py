@@ -1,5 +1,6 @@
-"""Dense gated feed-forward: down( silu(gate(x)) * up(x) ); optionally with biases on the three products and the
-clamped activation (`limit` > 0: g = min(gate, limit), u = clamp(up, -limit, limit), g sigmoid(1.702 g) (u + 1)).
+"""Dense gated feed-forward: down( silu(gate(x)) * up(x) ); optionally with biases on the three products and another
+activation: the clamped one (`limit` > 0: g = min(gate, limit), u = clamp(up, -limit, limit), g sigmoid(1.702 g) (u + 1))
+or gelu in its tanh form in silu's place (`activation` "gelu_tanh").
 
 gate and up are stacked into one [2I, H] matrix, gate rows first (reference:
 src/model/qwen2.cc:1413-1434 load, :1042-1048 forward; SiluMulFusedKernel
@@ -38,9 +39,14 @@ class BiasedDelta(LazyDelta):
 class DenseMlp(FeedForward):
     graph_safe = True
 
-    def __init__(self, hidden_size: int, width: int, init_std: float = 0.02, bias: bool = False, limit: float = 0.0):
+    def __init__(self, hidden_size: int, width: int, init_std: float = 0.02, bias: bool = False, limit: float = 0.0,
+                 activation: str = "silu"):
+        from .. import ops
         self.hidden_size, self.width, self.init_std = int(hidden_size), int(width), float(init_std)
-        self.bias, self.limit = bool(bias), float(limit)
+        if activation not in ("silu", "gelu_tanh") or limit < 0 or (limit and activation != "silu"):
+            raise ValueError(f"activation {activation!r} with limit {limit}: silu, gelu_tanh, or silu's clamped form by a limit")
+        self.bias = bool(bias)
+        self.form = ops.GLU_GELU_TANH if activation == "gelu_tanh" else float(limit)  # as the kernels name it
         self.w_gate_up = self.w_down = self.b_gate_up = self.b_down = None
 
     def param_specs(self) -> List[ParamSpec]:
@@ -63,7 +69,7 @@ class DenseMlp(FeedForward):
         """The result without the last product's bias: whoever adds the result to the stream adds `out_bias()` with
         it (`BiasedDelta`), so that the bias costs no pass of its own."""
         rt = ctx.rt
-        y = rt.linear(rt.gated_linear(x, self.w_gate_up, self.limit, self.b_gate_up), self.w_down)
+        y = rt.linear(rt.gated_linear(x, self.w_gate_up, self.form, self.b_gate_up), self.w_down)
         return y if self.b_down is None else BiasedDelta(y, self.b_down)
 
 

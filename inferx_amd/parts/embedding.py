@@ -12,7 +12,7 @@ from typing import List, Optional
 import torch
 
 from .. import ops
-from .base import Embedding, Head, ParamSpec, register_part
+from .base import EmbeddedRows, Embedding, Head, ParamSpec, register_part
 
 
 class TokenEmbedding(Embedding):
@@ -48,6 +48,11 @@ class TokenEmbedding(Embedding):
         h = ctx.rt.empty((ctx.num_tokens, self.hidden_size), torch.float32)
         ops.embed(h, self.weight, ctx.token_ids, self.scale)
         return h
+
+    def again(self, ctx, h):
+        if self.norm_eps is not None or self.streams is not None:
+            return super().again(ctx, h)
+        return EmbeddedRows(self.weight, ctx.token_ids, self.scale)
 
 
 class LinearHead(Head):

@@ -31,6 +31,11 @@ class DecoderModel:
             block = build_block(layer.block, layer.parts)
             self.blocks.append(block)
             self._part_specs += [(layer.parts[name], block.parts[name]) for name in layer.parts]
+        self.entries = []  # per schedule entry the part that the stream passes before it, or None
+        for entry in spec.schedule:
+            self.entries.append(None if entry.enter is None else build_part("entry", entry.enter))
+            if entry.enter is not None:
+                self._part_specs.append((entry.enter, self.entries[-1]))
         self.final_norm = build_part("norm", spec.final_norm)
         self.head = build_part("head", spec.head)
         self._part_specs += [(spec.final_norm, self.final_norm), (spec.head, self.head)]
@@ -71,6 +76,7 @@ class DecoderModel:
         for b in self.blocks:
             out.append(b)
             out += list(b.parts.values())
+        out += [e for e in self.entries if e is not None]
         for p in list(out):
             out += [s for s in getattr(p, "subparts", lambda: [])() if s is not None]
         return out
@@ -99,7 +105,10 @@ class DecoderModel:
         s = self.spec
         h = self.embedding.forward(ctx)
         pending = None
+        again = self.embedding.again(ctx, h) if any(e is not None and e.needs_embedding for e in self.entries) else None
         for i, entry in enumerate(s.schedule):
+            if self.entries[i] is not None:
+                pending = self.entries[i].forward(ctx, pending, again)
             pending = self.blocks[entry.layer].forward(ctx, h, pending, caches[i])
         rows = ctx.logits_rows
         if rows.numel() == 0:

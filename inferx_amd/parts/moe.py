@@ -14,7 +14,8 @@ neighbours, a group's score is its best expert's, and only experts of the best `
 Further: `score` "sigmoid" (an expert's score is the sigmoid of its own logit, not the softmax over all),
 `group_score` "top2" (a group's score is the sum of its two best experts'), and the activation "clamped_glu" with
 `limit` (and `shared_limit` for the shared expert): g = min(gate, limit), u = clamp(up, -limit, limit),
-g sigmoid(1.702 g) (u + 1).
+g sigmoid(1.702 g) (u + 1).  `router_bias`: a learned number per expert joins its score before anything else (with
+`renormalize` the weights are then the softmax over the chosen experts' biased scores alone).
 """
 from __future__ import annotations
 
@@ -58,7 +59,7 @@ class MoeFeedForward(FeedForward):
                  shared_gated: bool = True, renormalize: bool = False, routed_scale: float = 1.0,
                  init_std: float = 0.02, gated: bool = True, activation: Optional[str] = None, groups: int = 1,
                  groups_keep: int = 1, score: str = "softmax", group_score: str = "best", limit: float = 0.0,
-                 shared_limit: Optional[float] = None):
+                 shared_limit: Optional[float] = None, router_bias: bool = False):
         if not 0 < top_k <= num_experts:
             raise ValueError(f"top_k {top_k} must be between 1 and num_experts {num_experts}")
         if num_experts > 1024 or top_k > 32:
@@ -96,12 +97,15 @@ class MoeFeedForward(FeedForward):
             self.shared_width > 0 and self.shared_width % self.expert_width == 0
             and self.shared_width // self.expert_width <= 32 and self.shared_limit == self.limit) else 0
         self.w13_all = self.w2_all = None  # routed experts, then the shared expert's pieces
-        self.w_router = self.w13 = self.w2 = None
+        self.router_bias = bool(router_bias)
+        self.w_router = self.b_router = self.w13 = self.w2 = None
         self.w_shared_gate_up = self.w_shared_down = self.w_shared_gate = None
 
     def param_specs(self) -> List[ParamSpec]:
         H, mi, si, s = self.hidden_size, self.expert_width, self.shared_width, self.init_std
         specs = [ParamSpec("gate.weight", (self.num_experts, H), std=s)]
+        if self.router_bias:
+            specs.append(ParamSpec("gate.bias", (self.num_experts,), std=0.5))
         for e in range(self.num_experts):
             if self.gated:
                 specs.append(ParamSpec(f"experts.{e}.gate_proj.weight", (mi, H), std=s))
@@ -118,6 +122,8 @@ class MoeFeedForward(FeedForward):
     def bind(self, tensors, rt) -> None:
         E = self.num_experts
         self.w_router = tensors["gate.weight"].contiguous()
+        if self.router_bias:
+            self.b_router = tensors["gate.bias"].to(torch.float32).contiguous()
         parts = []
         for e in range(E):
             if self.gated:
@@ -153,7 +159,7 @@ class MoeFeedForward(FeedForward):
         topk_e = rt.empty((T, k), torch.int32)
         gate = rt.empty((T,), torch.float32) if self.w_shared_gate is not None else None
         ops.moe_route(x, self.w_router, self.w_shared_gate, topk_w, topk_e, gate, self.renormalize, self.routed_scale,
-                      always, self.groups, self.groups_keep, self.sigmoid_scores, self.group_top2)
+                      always, self.groups, self.groups_keep, self.sigmoid_scores, self.group_top2, self.b_router)
         return topk_w, topk_e, gate
 
     def _tile_rows(self, ctx, x) -> int:
@@ -234,7 +240,7 @@ class MoeFeedForward(FeedForward):
         tile_map = rt.empty((2 * ops.moe_max_tiles(T * k, E, tile_rows) + 1,), torch.int32) if tile_rows else None
         ops.moe_route_dispatch(None if norm else x, self.w_router, self.w_shared_gate, topk_w, topk_e, gate,
                                self.renormalize, self.routed_scale, offsets, rows, dest, tile_rows, tile_map, norm,
-                               self.groups, self.groups_keep, self.sigmoid_scores, self.group_top2)
+                               self.groups, self.groups_keep, self.sigmoid_scores, self.group_top2, self.b_router)
         return topk_w, topk_e, gate, offsets, rows, dest, tile_map
 
     def _routes_in_one_launch(self, tokens: int) -> bool:

@@ -11,6 +11,7 @@ import torch
 
 from .. import ops
 from .base import LazyDelta, Norm, ParamSpec, register_part
+from .branch_sum import BranchSum
 
 
 class RMSNorm(Norm):
@@ -59,6 +60,14 @@ class RMSNorm(Norm):
             delta = delta.materialize(ctx)
         ops.add_rmsnorm(h, delta, self.weight, out, self.eps, rows, self.groups)
         return out
+
+    def forward_pair(self, ctx, h, delta, other):
+        mine, its, total = self.rms_operands(), other.rms_operands(), BranchSum.of(delta)
+        if mine is None or its is None or mine[1] != its[1] or total is None:
+            return super().forward_pair(ctx, h, delta, other)
+        x, z = ctx.rt.empty(tuple(h.shape)), ctx.rt.empty(tuple(h.shape))
+        total.form(ctx, h, [(mine[0], x), (its[0], z)], mine[1])
+        return x, z
 
 
 class NormedDelta(LazyDelta):

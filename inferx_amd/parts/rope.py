@@ -23,6 +23,9 @@ index i,
 
 (fast waves stay, slow ones are stretched), and cosine and sine are both multiplied by `gain` = 0.1 ln(s) + 1.
 Which elements of a head a table's pair j turns is the business of the kernel that applies it.
+
+`widen(pairs)` lengthens the table with pairs of frequency zero (cosine 1, sine 0: they turn nothing), for an attention
+that arranges a head so that all of it is paired although a part of it is rotated.
 """
 from __future__ import annotations
 
@@ -59,7 +62,14 @@ class Rotary(PositionEncoding):
                 if self.theta == 1.0:
                     raise ValueError("a ramp over the frequencies needs a theta other than 1")
                 self.gain = 0.1 * math.log(float(self.scaling["factor"])) + 1.0
+        self.pairs = self.rotary_dim // 2  # of the table
         self.inv_freq = None
+
+    def widen(self, pairs: int) -> None:
+        """From now on (before `bind`) the table holds that many pairs."""
+        if pairs < self.rotary_dim // 2:
+            raise ValueError(f"a table of {pairs} pairs does not hold the {self.rotary_dim // 2} that are rotated")
+        self.pairs = int(pairs)
 
     def frequencies(self) -> torch.Tensor:
         d = self.rotary_dim
@@ -75,16 +85,17 @@ class Rotary(PositionEncoding):
                 f = f / factor * ramp + f * (1.0 - ramp)
             else:
                 f = f / factor
+        f = torch.cat([f, torch.zeros(self.pairs - d // 2, dtype=torch.float64)])
         return f.to(torch.float32)
 
     def bind(self, tensors, rt) -> None:
         self.inv_freq = self.frequencies().to(rt.device)
 
     def prepare(self, ctx):
-        key = ("rope", self.theta, self.rotary_dim, tuple(sorted(self.scaling.items())) if self.scaling else None)
+        key = ("rope", self.theta, self.rotary_dim, self.pairs, tuple(sorted(self.scaling.items())) if self.scaling else None)
         table = ctx.memo.get(key)
         if table is None:
-            table = ctx.rt.empty((ctx.num_tokens, self.rotary_dim // 2, 2), torch.float32)
+            table = ctx.rt.empty((ctx.num_tokens, self.pairs, 2), torch.float32)
             ops.rope_table(table, ctx.positions, self.inv_freq, self.gain)
             ctx.memo[key] = table
         return table
