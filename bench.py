@@ -37,6 +37,7 @@ feed-forward width, vocabulary and layers), both through the step function, at a
     python bench.py --workload bibevik [--sizes 1k,2k] [--only bibevik|dezudra]       # Bibevik beside Dezudra
     python bench.py --workload gosuvik [--sizes 1k,2k] [--only gosuvik|dezudra]       # Gosuvik beside Dezudra
     python bench.py --workload setopel [--sizes 1k,2k] [--only setopel|like_layers]   # Setopel beside other designs' like layers
+    python bench.py --workload zevivik [--sizes 1k,2k] [--only zevivik|like_layers]   # Zevivik beside other designs' like layers
 
 and a whole batch through the engine's loop (scheduler, portions, decode graphs as they come, sampling) at the same
 shape:
@@ -810,6 +811,102 @@ def run_setopel(args) -> int:
     return 0
 
 
+# Layer sizes for `--workload zevivik`: width, query heads and key/value heads of `dim` numbers (latent attention: `heads` heads
+# over a latent of `rank`), positions in a chunk, the dense feed-forward's width, experts, experts per token, their width and
+# the shared expert's, vocabulary
+ZEVIVIK_SIZES = {
+    "1k": dict(width=1024, heads=8, kv_heads=2, dim=128, rank=512, chunk=1024, ff=2816, experts=16, top=2, eff=704, shared=1408,
+               vocab=32000),
+    "2k": dict(width=2048, heads=16, kv_heads=4, dim=128, rank=512, chunk=1024, ff=5632, experts=32, top=4, eff=1408, shared=2816,
+               vocab=32000),
+    "4k": dict(width=4096, heads=32, kv_heads=8, dim=128, rank=512, chunk=1024, ff=11008, experts=64, top=4, eff=1408, shared=2816,
+               vocab=32000),
+}
+
+
+def run_zevivik(args) -> int:
+    """Prefill of one prompt and decode steps of a batch, through the step function, for the Zevivik design (an attention
+    layer with a dense feed-forward, then a loop of two passes over latent attention and two attention layers with experts)
+    and for a model put together from the like layers of the other designs, run in the same order at equal sizes: prenorm
+    layers with the Qwen2-MoE architecture's attention over a window of a chunk's size, Bibevik's latent attention with 64
+    rotated numbers, a dense feed-forward with silu, Bibevik's clamped experts with a shared one under a softmax router.
+    One JSON line; per size and model milliseconds and tokens a second of both phases, and Zevivik's time over the other's."""
+    import torch
+    from inferx_amd.config import LayerSpec, ModelSpec, PartSpec, ScheduleEntry, config_from_dict, linear_head, token_embedding
+    from inferx_amd.engine.runtime import Runtime
+
+    L = args.layers or 4
+    B, C, N = args.batch, args.prompt_len, args.prefill_tokens
+    rt = Runtime(args.dtype, "cuda:0")
+    gen = torch.Generator().manual_seed(1234)
+    out = {}
+
+    def specs(z):
+        W, H, G, D, R = z["width"], z["heads"], z["kv_heads"], z["dim"], z["rank"]
+        limit = 7.0
+        moe = {"kind": "moe", "expert": {"ff": z["eff"], "limit": limit}, "router": {"experts": z["experts"], "top": z["top"]},
+               "shared": {"ff": z["shared"], "limit": limit}}
+        attention = {"heads": H, "kv_heads": G, "dim": D, "vdim": D, "scale": D ** -0.5, "mask": {"size": z["chunk"]},
+                     "rot": {"dims": D, "base": 10000.0}}
+        latent = {"heads": H, "dim": D, "vdim": D, "kv_rank": R, "scale": D ** -0.5}
+        kinds = ["attention"] + [["latent_attention", "attention", "attention"][i % 3] for i in range(L - 1)]
+        loop = {"start": 1, "stop": L, "times": 2} if L > 1 else None
+        mine = {"architecture": "Zevivik", "vocab": z["vocab"], "width": W, "norm": {"eps": 1e-6}, "embedding": {"scale": 1.0},
+                "layers": [{"type": k, "mixer": attention if k == "attention" else latent,
+                            "mlp": {"kind": "dense", "ff": z["ff"]} if i == 0 else moe} for i, k in enumerate(kinds)]}
+        if loop:
+            mine["loop"] = loop
+        norm = PartSpec("rmsnorm", {"width": W, "eps": 1e-6})
+        named = lambda name: PartSpec("rmsnorm", {"width": W, "eps": 1e-6}, rename={"weight": name})
+        rope = lambda dims: PartSpec("rope", {"theta": 10000.0, "rotary_dim": dims})
+        mixers = {"attention": PartSpec("attention", {"hidden_size": W, "num_heads": H, "num_kv_heads": G, "head_dim": D,
+                                                      "position": rope(D), "window": z["chunk"], "qkv_bias": False}),
+                  "latent_attention": PartSpec("latent_attention", {"hidden_size": W, "num_heads": H, "head_dim": D, "rot_dim": 64,
+                                                                    "value_dim": D, "kv_rank": R, "position": rope(64)})}
+        dense = PartSpec("dense_mlp", {"hidden_size": W, "width": z["ff"]})
+        experts = PartSpec("moe", {"hidden_size": W, "num_experts": z["experts"], "top_k": z["top"], "expert_width": z["eff"],
+                                   "shared_width": z["shared"], "shared_gated": False, "renormalize": True,
+                                   "activation": "clamped_glu", "limit": limit})
+        layers = []
+        for i, k in enumerate(kinds):
+            at = lambda part, under: PartSpec(part.kind, part.params, prefix=f"l{i}.{under}.")
+            layers.append(LayerSpec("prenorm", {"mixer_norm": at(norm, "n1"), "mixer": at(mixers[k], "mix"),
+                                                "feed_forward_norm": at(norm, "n2"), "feed_forward": at(dense if i == 0 else experts, "mlp")}))
+        order = list(range(L)) + (list(range(1, L)) if loop else [])
+        like = ModelSpec(architecture="like layers", hidden_size=W, vocab_size=z["vocab"], max_positions=0, layers=layers,
+                         schedule=[ScheduleEntry(i) for i in order], embedding=token_embedding("embed", z["vocab"], W),
+                         final_norm=named("final.norm"), head=linear_head("head", z["vocab"], W))
+        return {"zevivik": config_from_dict(mine).model_spec(), "like_layers": like}
+
+    for name in [n for n in args.sizes.split(",") if n]:
+        z = ZEVIVIK_SIZES[name]
+        res = {}
+        for which, spec in specs(z).items():
+            if args.only and which != args.only:
+                continue
+            log(f"{name}: {which}")
+            pre, dec = _time_prefill_and_decode(args, rt, spec, z["vocab"], gen)
+            res[which] = {"prefill_ms": round(pre * 1e3, 3), "prefill_tokens_s": round(N / pre, 1),
+                          "decode_ms": round(dec * 1e3, 3), "decode_tokens_s": round(B / dec, 1)}
+            log(f"{name}: {which}: {res[which]}")
+        if len(res) == 2:
+            res["zevivik_over_like_layers"] = {
+                "prefill": round(res["zevivik"]["prefill_ms"] / res["like_layers"]["prefill_ms"], 3),
+                "decode": round(res["zevivik"]["decode_ms"] / res["like_layers"]["decode_ms"], 3)}
+        out[name] = dict(res, sizes=z)
+    first = out[next(iter(out))]
+    mine = first.get("zevivik") or next(iter(v for v in first.values() if isinstance(v, dict) and "decode_ms" in v))
+    print(json.dumps({
+        "metric": f"Zevivik decode tok/s @ batch {B} ({C}-token contexts), first size", "value": mine["decode_tokens_s"],
+        "unit": "tokens/s", "n_gpus": 1, "steps": args.steps, "warmup": args.warmup,
+        "ms_per_step": mine["decode_ms"], "higher_is_better": True, "scaling": "weak", "vs_baseline": None,
+        "dtype": "bf16" if args.dtype == "bfloat16" else "fp32", "data": "synthetic: seeded random weights and token ids",
+        "config": {"model": "Zevivik beside the like layers of other designs at equal sizes", "layers": L, "global_batch": B,
+                   "seq_len": C, "prefill_tokens": N, "parallelism": "single GPU", "page_size": PAGE},
+        "sizes": out}), flush=True)
+    return 0
+
+
 def run_pelalix(args) -> int:
     """Prefill of one prompt and decode steps of a batch, through the step function, for the Pelalix design and for
     the Qwen2-MoE architecture's dense layers (attention with rotation, RMS norms, the same gated feed-forward) at
@@ -893,7 +990,7 @@ def main() -> int:
     ap.add_argument("--scarce", action="store_true", help="offline: so few pages that sequences are preempted")
     ap.add_argument("--workload", default="decode",
                     choices=["decode", "mixed", "long", "mixed-small", "offline", "portion", "pelalix", "dezudra", "bibevik",
-                             "gosuvik", "setopel"],
+                             "gosuvik", "setopel", "zevivik"],
                     help="decode, mixed-small: the Qwen1.5-MoE-A2.7B shape (decode is the default); mixed, long: the "
                          "Qwen2-57B-A14B shape")
     ap.add_argument("--batch", type=int, default=8)
@@ -905,8 +1002,8 @@ def main() -> int:
     ap.add_argument("--prefill-context", type=int, default=0,
                     help="portion: tokens that the request has read before the timed portion")
     ap.add_argument("--shape", default="a27b", choices=["a27b", "57b"], help="portion: whose layer sizes")
-    ap.add_argument("--sizes", default="2k,4k", help="pelalix, dezudra, bibevik, gosuvik, setopel: which of the layer sizes " + ", ".join(PELALIX_SIZES))
-    ap.add_argument("--only", default="", help="bibevik, gosuvik, setopel: time one of the two models only (by its name)")
+    ap.add_argument("--sizes", default="2k,4k", help="pelalix, dezudra, bibevik, gosuvik, setopel, zevivik: which of the layer sizes " + ", ".join(PELALIX_SIZES))
+    ap.add_argument("--only", default="", help="bibevik, gosuvik, setopel, zevivik: time one of the two models only (by its name)")
     ap.add_argument("--prompt-len", type=int, default=PROMPT,
                     help="tokens of every request's prompt before it decodes (the context of the decode steps)")
     args = ap.parse_args()
@@ -914,9 +1011,9 @@ def main() -> int:
         print("bench.py: this engine runs on one GPU; --gpus N > 1 is not supported")
         return 2
     if args.steps is None:
-        args.steps = {"decode": 32, "mixed": 8, "long": 256, "mixed-small": 24, "offline": 0, "portion": 2, "pelalix": 32, "dezudra": 32, "bibevik": 32, "gosuvik": 32, "setopel": 32}[args.workload]
+        args.steps = {"decode": 32, "mixed": 8, "long": 256, "mixed-small": 24, "offline": 0, "portion": 2, "pelalix": 32, "dezudra": 32, "bibevik": 32, "gosuvik": 32, "setopel": 32, "zevivik": 32}[args.workload]
     if args.warmup is None:
-        args.warmup = {"decode": 4, "mixed": 2, "long": 4, "mixed-small": 4, "offline": 0, "portion": 1, "pelalix": 4, "dezudra": 4, "bibevik": 4, "gosuvik": 4, "setopel": 4}[args.workload]
+        args.warmup = {"decode": 4, "mixed": 2, "long": 4, "mixed-small": 4, "offline": 0, "portion": 1, "pelalix": 4, "dezudra": 4, "bibevik": 4, "gosuvik": 4, "setopel": 4, "zevivik": 4}[args.workload]
     if args.workload == "offline":
         return run_offline(args)
     if args.workload == "portion":
@@ -931,6 +1028,8 @@ def main() -> int:
         return run_gosuvik(args)
     if args.workload == "setopel":
         return run_setopel(args)
+    if args.workload == "zevivik":
+        return run_zevivik(args)
     if args.workload != "decode":
         return run_57b(args)
     if args.layers is None:

@@ -95,9 +95,9 @@ class BranchSum(LazyDelta):
     def materialize(self, ctx):
         shape = self._shape()
         if shape is None:
-            if not self.unformed:
-                return self.step  # (a vector alone)
-            total = self.unformed[0].materialize(ctx).to(torch.float32)
+            if not self.unformed:  # (a vector alone, for every token)
+                return None if self.step is None else self.step.to(torch.float32).expand(ctx.num_tokens, -1).contiguous()
+            total = self.unformed[0].materialize(ctx).to(torch.float32, copy=True)
             BranchSum(*self.unformed[1:]).entered(None, self.step).form(ctx, total)
             return total
         total = torch.zeros(shape, dtype=torch.float32, device=ctx.rt.device)

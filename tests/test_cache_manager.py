@@ -82,6 +82,51 @@ def test_window_rule_exactly():
     assert m.block_row("a", 0)[1] == -1
 
 
+def test_chunk_rule_exactly():
+    # page j is dead once (j + 1) * P <= cached - cached % C: the next position's chunk starts after it
+    m = CacheManager([GroupLayout(chunk=10)], [16], page_size=4, max_requests=1, max_seq_len=64)
+    m.add("a")
+    held = lambda: [j for j, p in enumerate(m.block_row("a", 0)) if p >= 0]
+    m.reserve("a", 24)
+    m.commit("a", 9)     # the next query, at 9, reads 0..9
+    assert held() == [0, 1, 2, 3, 4, 5]
+    m.commit("a", 1)     # at 10: its chunk starts at 10, pages 0 and 1 (0..7) are dead, page 2 holds 10 and 11
+    assert held() == [2, 3, 4, 5]
+    m.commit("a", 9)     # at 19: still 10..19
+    assert held() == [2, 3, 4, 5]
+    m.commit("a", 1)     # at 20: page 4 (16..19) is dead too
+    assert held() == [5]
+    keep = CacheManager([GroupLayout(chunk=10, release_passed=False)], [16], page_size=4, max_requests=1, max_seq_len=64)
+    keep.add("a")
+    keep.reserve("a", 24)
+    keep.commit("a", 24)
+    assert keep.pools[0].used_pages == 6
+    for c in (m, keep):
+        c.free("a")
+        c.check()
+        assert c.pools[0].used_pages == 0
+
+
+def test_a_chunked_group_takes_pages_as_the_steps_reach_them():
+    # chunks of 9, pages of 4, steps of at most 6 tokens: a pool of what a window of 9 needs never runs out
+    per_request = pages_for_window(9, 4, 1, 6)
+    m = CacheManager([GroupLayout(0), GroupLayout(chunk=9)], [32, per_request], page_size=4, max_requests=1, max_seq_len=128,
+                     max_step_tokens=6)
+    m.add("a")
+    assert m.reserve("a", 100) == RESERVE_OK
+    fed = 0
+    for n in [6, 1, 2, 5, 3, 6] * 4 + [6, 2]:
+        batch = build_step_batch(m, [("a", [1] * n, [])])
+        first = fed - fed % 9  # every key from the chunk's start on is on a page
+        assert batch.slots[1].min() >= 0 and all(m.block_row("a", 1)[j] >= 0 for j in range(first // 4, (fed + n - 1) // 4 + 1))
+        m.commit("a", n)
+        fed += n
+        m.check()
+    assert fed == 100 and m.pools[0].used_pages == 25 and m.pools[1].used_pages <= 3
+    m.free("a")
+    assert all(p.used_pages == 0 for p in m.pools)
+
+
 def test_a_windowed_group_may_keep_every_page():
     # the switch for differential tests: the same window, but passed pages stay until the request ends
     keep = CacheManager([GroupLayout(5, release_passed=False)], [16], page_size=4, max_requests=1, max_seq_len=64)
