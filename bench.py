@@ -815,11 +815,11 @@ def run_setopel(args) -> int:
 # over a latent of `rank`), positions in a chunk, the dense feed-forward's width, experts, experts per token, their width and
 # the shared expert's, vocabulary
 ZEVIVIK_SIZES = {
-    "1k": dict(width=1024, heads=8, kv_heads=2, dim=128, rank=512, chunk=1024, ff=2816, experts=16, top=2, eff=704, shared=1408,
+    "1k": dict(width=1024, heads=8, kv_heads=2, dim=128, rank=512, chunk=1280, ff=2816, experts=16, top=2, eff=704, shared=1408,
                vocab=32000),
-    "2k": dict(width=2048, heads=16, kv_heads=4, dim=128, rank=512, chunk=1024, ff=5632, experts=32, top=4, eff=1408, shared=2816,
+    "2k": dict(width=2048, heads=16, kv_heads=4, dim=128, rank=512, chunk=1280, ff=5632, experts=32, top=4, eff=1408, shared=2816,
                vocab=32000),
-    "4k": dict(width=4096, heads=32, kv_heads=8, dim=128, rank=512, chunk=1024, ff=11008, experts=64, top=4, eff=1408, shared=2816,
+    "4k": dict(width=4096, heads=32, kv_heads=8, dim=128, rank=512, chunk=1280, ff=11008, experts=64, top=4, eff=1408, shared=2816,
                vocab=32000),
 }
 

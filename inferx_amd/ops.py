@@ -1347,7 +1347,6 @@ def branch_norm(h: torch.Tensor, a: Optional[torch.Tensor] = None, b: Optional[t
     rows are normalised and h stays as it is."""
     T, W = h.shape
     _need(h.dtype == torch.float32, "the residual stream is float32 [T, W]")
-    dense = [t for t in (a, b) if t is not None]
     y = dest = topk_w = shared = gate = None
     k = 0
     if experts is not None:
@@ -1357,21 +1356,22 @@ def branch_norm(h: torch.Tensor, a: Optional[torch.Tensor] = None, b: Optional[t
               "the experts' rows do not fit")
         _is_i32(dest, T * k)
         _need(gate is None or (gate.dtype == torch.float32 and gate.numel() >= T), "the shared gate must be float32 [T]")
-        dense += [] if shared is None else [shared]
-    for t in dense:
-        _need(t.shape == h.shape, "a branch's result must have the shape of h")
-    outs = [o for _, o in norms]
-    types = {t.dtype for t in dense + outs + ([y] if y is not None else [])}
-    _need(len(types) <= 1, "the branches and the normalised rows must be of one type")
-    dtype = _dt(next(t for t in dense + outs + ([y] if y is not None else []))) if types else F32
     _need(len(norms) <= 2, "at most two norms")
+    (w1, o1), (w2, o2) = (*norms, (None, None), (None, None))[:2]
     n = T
     if rows is not None:
-        _need(len(norms) > 0, "picked rows are for a norm's result")
-        n = outs[0].shape[0]
+        _need(o1 is not None, "picked rows are for a norm's result")
+        n = o1.shape[0]
         _is_i32(rows, n)
-    for w, o in norms:
-        _need(w.numel() == W and o.shape == (n, W), "a norm's weight or result does not fit")
+    kind = None
+    for t, shape in ((a, h.shape), (b, h.shape), (shared, h.shape), (y, None), (o1, (n, W)), (o2, (n, W))):
+        if t is not None:
+            _need(shape is None or t.shape == shape, "a branch's result must have the shape of h, a norm's a row per row asked for")
+            _need(kind is None or t.dtype == kind, "the branches and the normalised rows must be of one type")
+            kind = t.dtype
+    dtype = F32 if kind is None else _CODE[kind]
+    for w in (w1, w2):
+        _need(w is None or w.numel() == W, "a norm's weight does not fit")
     for v in (bias, step):
         _need(v is None or v.numel() == W, "one number per column")
     table = ids = None
@@ -1383,8 +1383,7 @@ def branch_norm(h: torch.Tensor, a: Optional[torch.Tensor] = None, b: Optional[t
         _need(ids is not None or table_rows >= T, "a row per token, or ids")
         if ids is not None:
             _is_i32(ids, T)
-    code = lambda t: _i32(_dt(t) if t is not None else F32)
-    (w1, o1), (w2, o2) = (list(norms) + [(None, None), (None, None)])[:2]
+    code = lambda t: F32 if t is None else _dt(t)
     _call("ix_branch_norm", _ptr(h), _i32(dtype), _ptr(a), _ptr(b), _ptr(bias), code(bias), _ptr(y), _ptr(dest), _ptr(topk_w),
           _i32(k), _ptr(shared), _ptr(gate if shared is not None else None), _ptr(table), code(table), _ptr(ids),
           _i64(table_rows), _f32(scale), _ptr(step), code(step), _ptr(w1), code(w1), _ptr(o1), _ptr(w2), code(w2), _ptr(o2),
