@@ -1,7 +1,7 @@
 """Interfaces of the parts a layer is put together from, and their registries.
 
 A part is built from the parameters in its `PartSpec`, never from a config
-object, and does not know which model it is in.  Seven kinds:
+object, and does not know which model it is in.  The kinds:
 
   Embedding         forward(ctx) -> the residual stream h, float32 [T, hidden] (or [T, copies, hidden])
   Norm              forward(ctx, h, delta=None, rows=None) -> normed activations
